@@ -262,7 +262,7 @@ def compare_designs(args) -> int:
         for blk in runner.model.blocks:
             ff = getattr(blk, "feed_forward", None)
             if ff is not None and hasattr(ff, "num_experts"):
-                per_expert = (ff.w_gate_up.numel() + ff.w_down.numel()) // ff.num_experts * ff.w_down.element_size()
+                per_expert = (ff.w_in.numel() + ff.w_down.numel()) // ff.num_experts * ff.w_down.element_size()
                 used = ff.num_experts * (1.0 - (1.0 - ff.top_k / ff.num_experts) ** batch)
                 weights += (used - ff.top_k) * per_expert
         kv = batch * (fill + args.steps / 2) * sum(runner.bytes_per_block) / 16

@@ -18,12 +18,13 @@ int psamd_embed(void* stream, const int32_t* ids, const void* table, int table_d
                 int hidden, int vocab);
 
 // x = residual + delta, where delta is [rows, hidden] (delta_dtype) or n_partials float32 slices of that
-// shape, partial_stride elements apart (the partial sums of a K-split product).
+// shape, partial_stride elements apart (the partial sums of a K-split product); with delta_scale (float
+// [hidden] or NULL) x = residual + delta_scale * delta, column by column.
 // rows == NULL: residual[r] = x[r], out[r] = weight * rmsnorm(x[r]) for r < out_rows.
 // rows != NULL: out[i] = weight * rmsnorm(x[rows[i]]); residual untouched.
 int psamd_add_rmsnorm(void* stream, float* residual, const void* delta, int delta_dtype, int n_partials,
-                      int64_t partial_stride, const int32_t* rows, const void* weight, int weight_dtype, float eps,
-                      void* out, int act_dtype, int64_t out_rows, int hidden);
+                      int64_t partial_stride, const float* delta_scale, const int32_t* rows, const void* weight,
+                      int weight_dtype, float eps, void* out, int act_dtype, int64_t out_rows, int hidden);
 
 // out[t, c] = act(gate_up[t, c]) * gate_up[t, inter + c]; gate: 0 = SiLU, 1 = ReLU, 2 = GELU (tanh form).
 int psamd_swiglu(void* stream, const void* gate_up, void* out, int act_dtype, int64_t tokens, int inter, int gate);
@@ -58,9 +59,10 @@ int psamd_qk_prepare_kv_append(void* stream, void* qkv, int act_dtype, int64_t t
                                const float* q_weight, const float* k_weight, int v_from_k, void* kv,
                                const int32_t* write_slot, int q_weight_per_head);
 
-// residual[r] += delta[r]; delta as for psamd_add_rmsnorm (one tensor in delta_dtype, or n_partials float32 slices).
+// residual[r] += scale * delta[r] + row; delta as for psamd_add_rmsnorm (one tensor in delta_dtype, or n_partials
+// float32 slices); scale and row float32 [hidden] or NULL (1 and 0).
 int psamd_residual_add(void* stream, float* residual, const void* delta, int delta_dtype, int n_partials,
-                       int64_t partial_stride, int64_t rows, int hidden);
+                       int64_t partial_stride, int64_t rows, int hidden, const float* scale, const float* row);
 // x[r, c] = x[r, c] * factor + row[c] (row may be NULL) on a float32 tensor [rows, hidden].
 int psamd_stream_affine(void* stream, float* x, int64_t rows, int hidden, float factor, const float* row);
 // out[r] = [a[r], b[r]] in act_dtype, a and b float32 [rows, hidden].
@@ -68,20 +70,31 @@ int psamd_concat_to_activation(void* stream, const float* a, const float* b, voi
                                int hidden);
 
 // One small product per head: out[t, h, n] = sum_k x[t, h, k] * w[h, n, k], float accumulation. Row t of
-// x starts at x + t * x_row, its head h at + h * x_head (elements), likewise out; w is [H, N, K], dense.
+// x starts at x + t * x_row, its head h at + h * x_head (elements), likewise out and gate; w is [H, N, K], dense.
+// gate (or NULL, in x's dtype): out[t, h, n] is multiplied by sigmoid(gate[t, h, n]).
 int psamd_heads_linear(void* stream, const void* x, int x_dtype, int64_t x_row, int x_head, const void* w, int w_dtype,
-                       void* out, int out_dtype, int64_t out_row, int out_head, int64_t M, int H, int N, int K);
+                       void* out, int out_dtype, int64_t out_row, int out_head, int64_t M, int H, int N, int K, const void* gate,
+                       int64_t gate_row, int gate_head);
 
-// Latent attention, one compressed vector per token. Row t of `in` is [hq heads x (dim + rot) | rank | rot]:
-// the compressed part is divided by its root mean square (eps inside the root) and multiplied by norm_w
-// (float [rank]), the shared key part and every head's last `rot` query dimensions are rotated pair by
-// pair, (2i, 2i + 1) by table[positions[t]][i] = (cos, sin). The page of kv ([blocks, 2, 1, 16 * slots])
-// gets the key [compressed | rotated part | zeros] and, transposed, the value [compressed | zeros];
-// q_lat[t, h] (slots wide) gets the rotated query part at [rank, rank + rot) and zeros behind it, and
-// is left alone in front: that is where the product of the head's other dimensions goes.
-int psamd_latent_kv_append(void* stream, const void* in, int64_t in_row, void* q_lat, int act_dtype, int64_t tokens,
-                           int hq, int dim, int rot, int rank, int slots, const int32_t* positions, const float* table,
-                           const float* norm_w, float eps, void* kv, const int32_t* write_slot);
+// Latent attention, one compressed vector per token. Row t of `low` is [rank | rot]: the compressed part is
+// divided by its root mean square (eps inside the root) and multiplied by norm_w (float [rank]), the
+// shared key part is rotated pair by pair by table[positions[t]][i] = (cos, sin), partners (2i, 2i + 1)
+// or, with `halves`, (i, i + rot/2). The page of kv ([blocks, 2, 1, 16 * slots]) gets the key
+// [compressed | rotated part | zeros] and, transposed, the value [compressed | zeros].
+// c_in (or NULL), rows c_row apart: the queries' own latent, normed the same way (c_norm_w) into c_out [tokens, c_rank].
+// q (or NULL), rows of hq heads x (dim + rot): q_lat[t, h] (slots wide) gets the head's last `rot` dimensions,
+// rotated, at [rank, rank + rot) and zeros behind them, and is left alone in front: that is where the
+// product of the head's other dimensions goes.
+int psamd_latent_kv_append(void* stream, const void* low, int64_t low_row, const void* c_in, int64_t c_row, int c_rank,
+                           const float* c_norm_w, void* c_out, const void* q, int64_t q_row, void* q_lat, int act_dtype,
+                           int64_t tokens, int hq, int dim, int rot, int rank, int slots, int halves,
+                           const int32_t* positions, const float* table, const float* norm_w, float eps, void* kv,
+                           const int32_t* write_slot);
+// The whole of q_lat from the heads' queries: [w_fold[h] . q[:dim] | rotated q[dim:] | zeros], w_fold [hq, rank, dim].
+// With dim 0 the front may be left alone: the caller zeroes it.
+int psamd_latent_query(void* stream, const void* q, int64_t q_row, const void* w_fold, void* q_lat, int act_dtype,
+                       int64_t tokens, int hq, int dim, int rot, int rank, int slots, int halves, const int32_t* positions,
+                       const float* table);
 
 // A causal convolution per channel over each item's tokens, continued from the item's state:
 // u[t, c] = conv_b[c] + sum_j conv_w[c, j] * v(t - (taps - 1) + j, c) with v(s, c) = in[s, c] + in_bias[c]
@@ -109,20 +122,24 @@ int psamd_gated_scan(void* stream, const float* gates, const float* gate_b, cons
 // Mixture of experts. Router: z = x w_router^T in float (x in x_dtype, w_router float [E, K]), score =
 // sigmoid(z); chosen[t, :] = the top largest scores' experts (lower index among equals, largest
 // first), weight[t, :] = those scores. bias (float [experts] or NULL) is added to z first. mode 1: the
-// choice is by z itself and the weights are the softmax over the chosen z alone.
+// choice is by z itself and the weights are the softmax over the chosen z alone. groups > 0 (mode 0): the
+// experts form that many equal runs of neighbours, a run's score is the sum of its two largest scores,
+// and only experts of the `keep` best runs can be chosen. The weights are multiplied by factor.
 int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_router, int32_t* chosen, float* weight,
-                    int64_t tokens, int K, int experts, int top, const float* bias, int mode);
+                    int64_t tokens, int K, int experts, int top, const float* bias, int mode, int groups, int keep, float factor);
 // The same choice from logits that a product has written (float [tokens, experts]).
 int psamd_moe_topk(void* stream, const float* logits, int32_t* chosen, float* weight, int64_t tokens, int experts,
-                   int top, const float* bias, int mode);
+                   int top, const float* bias, int mode, int groups, int keep, float factor);
 // Experts, one (token, choice) pair at a time: h = weight[t, j] * x[t]; g = min(gate h, limit), u =
 // clamp(up h, -limit, limit); act[t * top + j] = g * sigmoid(gate_alpha * g) * (u + up_shift);
-// out[j][t] = down act (float). w_gate_up is [E, 2F, K] (gate rows, then up rows), w_down [E, K, F].
-// weight_on_output: h = x[t] and out[j][t] = weight[t, j] * down act instead.
+// out[j][t] = down act (float). w_in is [E, 2F, K] (gate rows, then up rows), w_down [E, K, F].
+// weight_on_output: h = x[t] and out[j][t] = weight[t, j] * down act instead. kind 1: no gate, act = max(up h, 0)^2,
+// w_in is [E, F, K]. into_stream: out is [tokens, K] and every pair adds its output into it, times col_scale
+// (float [K] or NULL), with float atomics.
 int psamd_moe_experts_rows(void* stream, const void* x, const int32_t* chosen, const float* weight,
-                           const void* w_gate_up, const void* w_down, void* act, float* out, int dtype,
+                           const void* w_in, const void* w_down, void* act, float* out, int dtype,
                            int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
-                           float up_shift, int weight_on_output);
+                           float up_shift, int weight_on_output, int kind, int into_stream, const float* col_scale);
 
 // The same for bfloat16 with the pairs sorted by expert and every expert's pairs run through its
 // matrices in tiles on the matrix cores. ints: scratch of pairs + 3 * psamd_moe_grouped_max_tiles(pairs,
@@ -130,13 +147,14 @@ int psamd_moe_experts_rows(void* stream, const void* x, const int32_t* chosen, c
 int psamd_moe_grouped_tile_rows(int64_t pairs, int experts);
 int psamd_moe_grouped_max_tiles(int64_t pairs, int experts);
 int psamd_moe_experts_grouped(void* stream, const void* x, const int32_t* chosen, const float* weight,
-                              const void* w_gate_up, const void* w_down, void* act, float* out, int32_t* ints,
+                              const void* w_in, const void* w_down, void* act, float* out, int32_t* ints,
                               int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
-                              float up_shift, int grouped_already, int weight_on_output);
+                              float up_shift, int grouped_already, int weight_on_output, int kind, int into_stream,
+                              const float* col_scale);
 // psamd_moe_topk and the sorting of the pairs into `ints` in one workgroup, for up to 64 tokens;
 // psamd_moe_experts_grouped is then called with grouped_already = 1 and the same `ints`.
 int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, float* weight, int32_t* ints, int64_t tokens,
-                         int experts, int top, const float* bias, int mode);
+                         int experts, int top, const float* bias, int mode, int groups, int keep, float factor);
 // out[t, :] *= sigmoid(x[t] . w) for float out [tokens, out_hidden], x [tokens, hidden] in act_dtype, w float [hidden].
 int psamd_row_gate(void* stream, float* out, const void* x, int act_dtype, const float* w, int64_t tokens, int out_hidden,
                    int hidden);
@@ -275,13 +293,15 @@ int psamd_qkv_rope_append(void* stream, const void* x, const void* w, void* qkv_
                           const int32_t* write_slot);
 
 // Small steps without a norm kernel and without partial slices to add up (bfloat16, M <= 16):
-// the products that feed the residual stream add into it (psamd_linear_skinny_add: float atomics,
+// the products that feed the residual stream add into it (psamd_linear_skinny_add: float atomics, each
+// column times col_scale [n_out] where that is given,
 // K split over workgroups; the order of the additions differs from run to run), and the products
 // that read the normalized stream (q/k/v, gate/up, the output matrix) take rows of the float32
 // residual and apply the RMS norm themselves (weight norm_w, bfloat16 or float32; statistics in
 // 32-bit, eps inside the root). psamd_normed_supports: whether they take M tokens of width K.
 int psamd_normed_supports(int M, int K);
-int psamd_linear_skinny_add(void* stream, const void* x, const void* w, float* out, int M, int n_out, int K);
+int psamd_linear_skinny_add(void* stream, const void* x, const void* w, float* out, int M, int n_out, int K,
+                            const float* col_scale);
 int psamd_linear_normed(void* stream, const float* resid, const int32_t* rows, const void* norm_w, int norm_w_dtype,
                         float eps, const void* w, void* out, int out_dtype, int M, int n_out, int K, int epilogue);
 int psamd_qkv_rope_append_normed(void* stream, const float* resid, const void* norm_w, int norm_w_dtype, float eps,

@@ -37,11 +37,12 @@ __global__ void embed_kernel(const int32_t* __restrict__ ids, const W* __restric
 // Rows up to kCache * kThreads wide stay in registers between the two passes, and all loads
 // of a pass are independent of each other (clamped addresses, no branches around them), so
 // they are in flight together: with one row per block the kernel is pure latency.
-template <typename A, typename DT, int kThreads, int kCache>
+// SCALED: the slices' sum is multiplied by delta_scale[column] before it is added.
+template <typename A, typename DT, int kThreads, int kCache, bool SCALED>
 __global__ __launch_bounds__(kThreads) void add_rmsnorm_kernel(
     float* __restrict__ residual, const DT* __restrict__ delta, int n_partials, int64_t partial_stride,
-    const int32_t* __restrict__ rows, const void* __restrict__ weight, int weight_dtype, float eps,
-    A* __restrict__ out, int hidden) {
+    const float* __restrict__ delta_scale, const int32_t* __restrict__ rows, const void* __restrict__ weight,
+    int weight_dtype, float eps, A* __restrict__ out, int hidden) {
   __shared__ float scratch[kThreads / kWave];
   const int64_t src = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
   float* r = residual + src * hidden;
@@ -51,13 +52,14 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_kernel(
   const int np = delta != nullptr ? n_partials : 0;
 
   if (hidden <= kCache * kThreads) {
-    float v[kCache], wv[kCache];
+    float v[kCache], wv[kCache], add[SCALED ? kCache : 1];
     int idx[kCache];
 #pragma unroll
     for (int j = 0; j < kCache; ++j) {
       idx[j] = min(static_cast<int>(threadIdx.x) + j * kThreads, hidden - 1);
       v[j] = r[idx[j]];
       wv[j] = load_as_float(weight, weight_dtype, idx[j]);
+      if (SCALED) add[j] = 0.f;
     }
     for (int p = 0; p < np; ++p) {
       const DT* dp = d0 + p * partial_stride;
@@ -65,7 +67,11 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_kernel(
 #pragma unroll
       for (int j = 0; j < kCache; ++j) t[j] = to_float<DT>(dp[idx[j]]);
 #pragma unroll
-      for (int j = 0; j < kCache; ++j) v[j] += t[j];
+      for (int j = 0; j < kCache; ++j) (SCALED ? add[j] : v[j]) += t[j];
+    }
+    if (SCALED) {
+#pragma unroll
+      for (int j = 0; j < kCache; ++j) v[j] = fmaf(delta_scale[idx[j]], add[j], v[j]);
     }
     float ss = 0.f;
 #pragma unroll
@@ -86,9 +92,9 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_kernel(
   }
 
   auto value = [&](int i) {
-    float x = r[i];
+    float x = SCALED ? 0.f : r[i];
     for (int p = 0; p < np; ++p) x += to_float<DT>(d0[p * partial_stride + i]);
-    return x;
+    return SCALED ? fmaf(delta_scale[i], x, r[i]) : x;
   };
   float ss = 0.f;
   for (int i = threadIdx.x; i < hidden; i += kThreads) {
@@ -107,11 +113,11 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_kernel(
 // The same operation for bfloat16 activations and rows that are a multiple of 8 wide: every
 // thread owns runs of 8 consecutive elements, moved as 16- and 32-byte accesses. kIter runs
 // per thread stay in registers (hidden <= 8 * kThreads * kIter).
-template <typename DT, int kThreads, int kIter>
+template <typename DT, int kThreads, int kIter, bool SCALED>
 __global__ __launch_bounds__(kThreads) void add_rmsnorm_vec8_kernel(
     float* __restrict__ residual, const DT* __restrict__ delta, int n_partials, int64_t partial_stride,
-    const int32_t* __restrict__ rows, const void* __restrict__ weight, int weight_dtype, float eps,
-    bf16_t* __restrict__ out, int hidden) {
+    const float* __restrict__ delta_scale, const int32_t* __restrict__ rows, const void* __restrict__ weight,
+    int weight_dtype, float eps, bf16_t* __restrict__ out, int hidden) {
   __shared__ float scratch[kThreads / kWave];
   const int64_t src = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
   float* r = residual + src * hidden;
@@ -131,6 +137,15 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_vec8_kernel(
     const float4 b = *reinterpret_cast<const float4*>(r + e + 4);
     v[j][0] = a.x; v[j][1] = a.y; v[j][2] = a.z; v[j][3] = a.w;
     v[j][4] = b.x; v[j][5] = b.y; v[j][6] = b.z; v[j][7] = b.w;
+    float own[8];
+    float* acc = SCALED ? own : v[j];             // what the slices are added to
+    float4 sa, sb;
+    if (SCALED) {
+      sa = *reinterpret_cast<const float4*>(delta_scale + e);
+      sb = *reinterpret_cast<const float4*>(delta_scale + e + 4);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) own[i] = 0.f;
+    }
     for (int p = 0; p < np; ++p) {
       const DT* dp = d0 + p * partial_stride + e;
       if (sizeof(DT) == 2) {
@@ -138,8 +153,8 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_vec8_kernel(
         const uint32_t w4[4] = {q.x, q.y, q.z, q.w};
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          v[j][2 * i] += __uint_as_float(w4[i] << 16);
-          v[j][2 * i + 1] += __uint_as_float(w4[i] & 0xffff0000u);
+          acc[2 * i] += __uint_as_float(w4[i] << 16);
+          acc[2 * i + 1] += __uint_as_float(w4[i] & 0xffff0000u);
         }
       } else {
         // Up to eight slices are asked for together (one trip to memory, not one per slice) and
@@ -154,12 +169,17 @@ __global__ __launch_bounds__(kThreads) void add_rmsnorm_vec8_kernel(
 #pragma unroll
         for (int u = 0; u < 8; ++u) {
           if (p + u < np) {
-            v[j][0] += x0[u].x; v[j][1] += x0[u].y; v[j][2] += x0[u].z; v[j][3] += x0[u].w;
-            v[j][4] += x1[u].x; v[j][5] += x1[u].y; v[j][6] += x1[u].z; v[j][7] += x1[u].w;
+            acc[0] += x0[u].x; acc[1] += x0[u].y; acc[2] += x0[u].z; acc[3] += x0[u].w;
+            acc[4] += x1[u].x; acc[5] += x1[u].y; acc[6] += x1[u].z; acc[7] += x1[u].w;
           }
         }
         p += 7;
       }
+    }
+    if (SCALED) {
+      const float sc[8] = {sa.x, sa.y, sa.z, sa.w, sb.x, sb.y, sb.z, sb.w};
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[j][i] = fmaf(sc[i], own[i], v[j][i]);
     }
     if (cidx < chunks) {
 #pragma unroll
@@ -593,14 +613,18 @@ __global__ __launch_bounds__(256) void rope_norm_kv_append_kernel(
 
 // ------------------------------------------------------------------ sums and copies of the stream
 
-// residual += delta, where delta is one tensor or n_partials float32 slices (summed in ascending order).
+// residual += scale * delta + row, where delta is one tensor or n_partials float32 slices (summed in ascending
+// order); scale and row are [hidden] or null (1 and 0).
 template <typename DT>
 __global__ void residual_add_kernel(float* __restrict__ residual, const DT* __restrict__ delta, int n_partials,
-                                    int64_t partial_stride, int64_t n) {
+                                    int64_t partial_stride, int64_t n, const float* __restrict__ scale,
+                                    const float* __restrict__ row, int hidden) {
   for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < n;
        i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
-    float x = residual[i];
+    float x = scale != nullptr ? 0.f : residual[i];
     for (int p = 0; p < n_partials; ++p) x += to_float<DT>(delta[p * partial_stride + i]);
+    if (scale != nullptr) x = fmaf(scale[i % hidden], x, residual[i]);
+    if (row != nullptr) x += row[i % hidden];
     residual[i] = x;
   }
 }
@@ -649,7 +673,7 @@ int psamd_embed(void* stream, const int32_t* ids, const void* table, int table_d
 }
 
 int psamd_add_rmsnorm(void* stream, float* residual, const void* delta, int delta_dtype, int n_partials,
-                      int64_t partial_stride, const int32_t* rows, const void* weight, int weight_dtype, float eps,
+                      int64_t partial_stride, const float* delta_scale, const int32_t* rows, const void* weight, int weight_dtype, float eps,
                       void* out, int act_dtype, int64_t out_rows, int hidden) {
   PSAMD_REQUIRE(out_rows >= 0 && hidden > 0, "bad sizes");
   PSAMD_REQUIRE(weight_dtype == kF32 || weight_dtype == kBF16, "weight dtype must be float32 or bfloat16");
@@ -660,17 +684,20 @@ int psamd_add_rmsnorm(void* stream, float* residual, const void* delta, int delt
   hipStream_t s = static_cast<hipStream_t>(stream);
   constexpr int kThreads = 256, kCache = 16;
   const dim3 grid(static_cast<unsigned>(out_rows)), block(kThreads);
-#define PSAMD_NORM(A_, D_)                                                                                      \
-  add_rmsnorm_kernel<A_, D_, kThreads, kCache><<<grid, block, 0, s>>>(                                          \
-      residual, static_cast<const D_*>(delta), n_partials, partial_stride, rows, weight, weight_dtype, eps, \
-      static_cast<A_*>(out), hidden)
+  const bool scaled = delta != nullptr && delta_scale != nullptr;
+#define PSAMD_NORM_AS(A_, D_, S_)                                                                               \
+  add_rmsnorm_kernel<A_, D_, kThreads, kCache, S_><<<grid, block, 0, s>>>(                                      \
+      residual, static_cast<const D_*>(delta), n_partials, partial_stride, delta_scale, rows, weight,           \
+      weight_dtype, eps, static_cast<A_*>(out), hidden)
+#define PSAMD_NORM(A_, D_) do { if (scaled) PSAMD_NORM_AS(A_, D_, true); else PSAMD_NORM_AS(A_, D_, false); } while (0)
   const bool delta_f32 = delta == nullptr || delta_dtype == kF32;
   if (act_dtype == kBF16 && hidden % 8 == 0 && hidden <= 8 * kThreads * 4) {
     bf16_t* o16 = static_cast<bf16_t*>(out);
-#define PSAMD_NORM8(D_, IT_)                                                                                 \
-  add_rmsnorm_vec8_kernel<D_, kThreads, IT_><<<grid, block, 0, s>>>(                                         \
-      residual, static_cast<const D_*>(delta), n_partials, partial_stride, rows, weight, weight_dtype, eps, \
-      o16, hidden)
+#define PSAMD_NORM8_AS(D_, IT_, S_)                                                                          \
+  add_rmsnorm_vec8_kernel<D_, kThreads, IT_, S_><<<grid, block, 0, s>>>(                                     \
+      residual, static_cast<const D_*>(delta), n_partials, partial_stride, delta_scale, rows, weight,        \
+      weight_dtype, eps, o16, hidden)
+#define PSAMD_NORM8(D_, IT_) do { if (scaled) PSAMD_NORM8_AS(D_, IT_, true); else PSAMD_NORM8_AS(D_, IT_, false); } while (0)
     const int iters = static_cast<int>(ceil_div(hidden / 8, kThreads));
     if (delta_f32) {
       if (iters <= 1) PSAMD_NORM8(float, 1); else if (iters <= 2) PSAMD_NORM8(float, 2); else PSAMD_NORM8(float, 4);
@@ -678,6 +705,7 @@ int psamd_add_rmsnorm(void* stream, float* residual, const void* delta, int delt
       if (iters <= 1) PSAMD_NORM8(bf16_t, 1); else if (iters <= 2) PSAMD_NORM8(bf16_t, 2); else PSAMD_NORM8(bf16_t, 4);
     }
 #undef PSAMD_NORM8
+#undef PSAMD_NORM8_AS
     return check_launch("psamd_add_rmsnorm");
   }
   if (act_dtype == kBF16) {
@@ -688,6 +716,7 @@ int psamd_add_rmsnorm(void* stream, float* residual, const void* delta, int delt
     return fail("psamd_add_rmsnorm: activation dtype must be float32 or bfloat16");
   }
 #undef PSAMD_NORM
+#undef PSAMD_NORM_AS
   return check_launch("psamd_add_rmsnorm");
 }
 
@@ -846,9 +875,10 @@ int psamd_rope_norm_kv_append(void* stream, void* qkv, int act_dtype, int64_t to
                                     nullptr, nullptr, nullptr, 0, kv, write_slot, 0);
 }
 
-// residual[r] += delta[r] (delta as for psamd_add_rmsnorm: one tensor in delta_dtype or float32 slices).
+// residual[r] += scale * delta[r] + row (delta as for psamd_add_rmsnorm: one tensor in delta_dtype or float32 slices;
+// scale and row float32 [hidden] or NULL).
 int psamd_residual_add(void* stream, float* residual, const void* delta, int delta_dtype, int n_partials,
-                       int64_t partial_stride, int64_t rows, int hidden) {
+                       int64_t partial_stride, int64_t rows, int hidden, const float* scale, const float* row) {
   PSAMD_REQUIRE(rows >= 0 && hidden > 0 && n_partials >= 1 && delta != nullptr, "bad sizes");
   PSAMD_REQUIRE(n_partials == 1 || delta_dtype == kF32, "partial sums are float32");
   if (rows == 0) return 0;
@@ -857,10 +887,10 @@ int psamd_residual_add(void* stream, float* residual, const void* delta, int del
   const int blocks = static_cast<int>(std::min<int64_t>(ceil_div(n, 256), 65536));
   if (delta_dtype == kBF16) {
     residual_add_kernel<bf16_t><<<dim3(blocks), dim3(256), 0, s>>>(residual, static_cast<const bf16_t*>(delta), n_partials,
-                                                                  partial_stride, n);
+                                                                  partial_stride, n, scale, row, hidden);
   } else if (delta_dtype == kF32) {
     residual_add_kernel<float><<<dim3(blocks), dim3(256), 0, s>>>(residual, static_cast<const float*>(delta), n_partials,
-                                                                 partial_stride, n);
+                                                                 partial_stride, n, scale, row, hidden);
   } else {
     return fail("psamd_residual_add: delta dtype must be float32 or bfloat16");
   }

@@ -3,7 +3,8 @@
 // What latent attention needs twice (a head's query folded into the compressed space, and the
 // compressed result unfolded into the head's values) and what a recurrence with block-diagonal
 // gate matrices needs once. Rows of x and out are strided, so that a head's operand may sit
-// inside a wider row and its result may land inside another.
+// inside a wider row and its result may land inside another. Optionally every result is multiplied by
+// sigmoid(gate[t, h, n]), the gate's rows in the same element type (an output gate on attention's heads).
 //
 // Two forms. LDS-tiled FMA with float accumulation for any element types, the 32-bit path's
 // product: k is summed in ascending order whatever the number of tokens, so a token's 32-bit
@@ -20,7 +21,8 @@ namespace psamd {
 template <typename TX, typename TW, typename TO>
 __global__ __launch_bounds__(256) void heads_linear_kernel(const TX* __restrict__ x, int64_t x_row, int x_head,
                                                            const TW* __restrict__ w, TO* __restrict__ out, int64_t o_row,
-                                                           int o_head, int64_t M, int N, int K) {
+                                                           int o_head, int64_t M, int N, int K, const TX* __restrict__ gate,
+                                                           int64_t g_row, int g_head) {
   constexpr int BM = 64, BN = 64, BK = 16;
   __shared__ float xs[BK][BM + 1];
   __shared__ float wsm[BK][BN + 1];
@@ -64,7 +66,10 @@ __global__ __launch_bounds__(256) void heads_linear_kernel(const TX* __restrict_
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) out[m * o_row + n] = from_float<TO>(acc[i][j]);
+      if (n >= N) continue;
+      float v = acc[i][j];
+      if (gate != nullptr) v *= 1.f / (1.f + expf(-to_float<TX>(gate[m * g_row + static_cast<int64_t>(h) * g_head + n])));
+      out[m * o_row + n] = from_float<TO>(v);
     }
   }
 }
@@ -77,7 +82,8 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 template <int NT>
 __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const bf16_t* __restrict__ x, int64_t x_row, int x_head,
                                                                 const bf16_t* __restrict__ w, bf16_t* __restrict__ out,
-                                                                int64_t o_row, int o_head, int64_t M, int N, int K) {
+                                                                int64_t o_row, int o_head, int64_t M, int N, int K,
+                                                                const bf16_t* __restrict__ gate, int64_t g_row, int g_head) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
   const int h = blockIdx.z;
@@ -107,21 +113,26 @@ __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const bf16_t* __
   const int64_t m = m0 + r;
   if (m >= M) return;
   bf16_t* o = out + static_cast<int64_t>(h) * o_head + m * o_row;
+  const bf16_t* gt = gate != nullptr ? gate + static_cast<int64_t>(h) * g_head + m * g_row : nullptr;
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
       const int n = n0 + nt * 16 + 4 * g + v;
-      if (n < N) o[n] = float_to_bf16(acc[nt][v]);
+      if (n >= N) continue;
+      float y = acc[nt][v];
+      if (gt != nullptr) y *= 1.f / (1.f + __expf(-bf16_to_float(gt[n])));
+      o[n] = float_to_bf16(y);
     }
 }
 
 template <typename T>
 static int launch_heads(hipStream_t s, const void* x, int64_t x_row, int x_head, const void* w, void* out, int64_t o_row,
-                        int o_head, int64_t M, int H, int N, int K) {
+                        int o_head, int64_t M, int H, int N, int K, const void* gate, int64_t g_row, int g_head) {
   const dim3 grid(static_cast<unsigned>(ceil_div(N, 64)), static_cast<unsigned>(ceil_div(M, 64)), static_cast<unsigned>(H));
   heads_linear_kernel<T, T, T><<<grid, dim3(256), 0, s>>>(static_cast<const T*>(x), x_row, x_head, static_cast<const T*>(w),
-                                                          static_cast<T*>(out), o_row, o_head, M, N, K);
+                                                          static_cast<T*>(out), o_row, o_head, M, N, K,
+                                                          static_cast<const T*>(gate), g_row, g_head);
   return check_launch("psamd_heads_linear");
 }
 
@@ -131,12 +142,13 @@ using namespace psamd;
 
 extern "C" int psamd_heads_linear(void* stream, const void* x, int x_dtype, int64_t x_row, int x_head, const void* w,
                                   int w_dtype, void* out, int out_dtype, int64_t out_row, int out_head, int64_t M, int H,
-                                  int N, int K) {
+                                  int N, int K, const void* gate, int64_t gate_row, int gate_head) {
   PSAMD_REQUIRE(M >= 0 && H > 0 && N > 0 && K > 0, "bad sizes");
   PSAMD_REQUIRE(H <= 65535 && ceil_div(M, 64) <= 65535, "too large for one launch");
   PSAMD_REQUIRE(x_head >= 0 && out_head >= 0 && x_row >= static_cast<int64_t>(H - 1) * x_head + K &&
                 out_row >= static_cast<int64_t>(H - 1) * out_head + N, "rows too short for their heads");
   PSAMD_REQUIRE(x_dtype == w_dtype && x_dtype == out_dtype, "x, w and out must have one dtype");
+  PSAMD_REQUIRE(gate == nullptr || (gate_head >= 0 && gate_row >= static_cast<int64_t>(H - 1) * gate_head + N), "gate rows too short");
   if (M == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (x_dtype == kBF16 && K % 8 == 0 && x_row % 8 == 0 && x_head % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
@@ -145,10 +157,10 @@ extern "C" int psamd_heads_linear(void* stream, const void* x, int x_dtype, int6
     const dim3 grid(static_cast<unsigned>(ceil_div(N, 16 * NT)), static_cast<unsigned>(ceil_div(M, 64)), static_cast<unsigned>(H));
     heads_linear_mfma_kernel<NT><<<grid, dim3(256), 0, s>>>(static_cast<const bf16_t*>(x), x_row, x_head,
                                                            static_cast<const bf16_t*>(w), static_cast<bf16_t*>(out), out_row,
-                                                           out_head, M, N, K);
+                                                           out_head, M, N, K, static_cast<const bf16_t*>(gate), gate_row, gate_head);
     return check_launch("psamd_heads_linear");
   }
-  if (x_dtype == kBF16) return launch_heads<bf16_t>(s, x, x_row, x_head, w, out, out_row, out_head, M, H, N, K);
-  if (x_dtype == kF32) return launch_heads<float>(s, x, x_row, x_head, w, out, out_row, out_head, M, H, N, K);
+  if (x_dtype == kBF16) return launch_heads<bf16_t>(s, x, x_row, x_head, w, out, out_row, out_head, M, H, N, K, gate, gate_row, gate_head);
+  if (x_dtype == kF32) return launch_heads<float>(s, x, x_row, x_head, w, out, out_row, out_head, M, H, N, K, gate, gate_row, gate_head);
   return fail("psamd_heads_linear: dtype must be float32 or bfloat16");
 }

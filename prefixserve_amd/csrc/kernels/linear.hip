@@ -176,11 +176,13 @@ constexpr int skinny_depth(int mt, int rt) { return mt == 1 ? 8 : (mt * rt <= 2 
 
 // ATOMIC (float32 output, plain epilogue): every K-slice adds its partial sums into the one
 // out[M][n_out] with float atomics that return nothing, instead of writing a slice of its own:
-// out is the residual stream, and no kernel has to add the slices up afterwards. The order of
+// out is the residual stream, and no kernel has to add the slices up afterwards (each multiplied by
+// col_scale[column] first, where that is given). The order of
 // the additions, and with it the last bit of the sums, differs from run to run.
 template <int MT, int RT, int WV, bool SWIGLU, bool SPLIT, typename TO, int U = skinny_depth(MT, RT), bool ATOMIC = false>
 __global__ __launch_bounds__(64 * WV) void skinny_mfma_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
-                                                          TO* __restrict__ out, int M, int n_out, int K, int act = 0) {
+                                                          TO* __restrict__ out, int M, int n_out, int K, int act = 0,
+                                                          const float* __restrict__ col_scale = nullptr) {
   constexpr int NACC = SWIGLU ? 2 * MT : MT;
   __shared__ f32x4 red[SPLIT ? WV : 1][NACC][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -278,7 +280,7 @@ __global__ __launch_bounds__(64 * WV) void skinny_mfma_kernel(const bf16_t* __re
     for (int v = 0; v < 4; ++v) {
       const int n = (tile0 + rt) * 16 + 4 * g + v;
       if (n >= n_out) continue;
-      if constexpr (ATOMIC) add_to(dst + n, sum[v]);
+      if constexpr (ATOMIC) add_to(dst + n, col_scale != nullptr ? col_scale[n] * sum[v] : sum[v]);
       else dst[n] = from_float<TO>(sum[v]);
     }
   };
@@ -406,7 +408,8 @@ __device__ __forceinline__ float stage_scale(const Tokens& tk, const float* ss, 
 // out[M][n_out] (see skinny_mfma_kernel).
 template <int RT, int ROWS, bool SWIGLU, typename TO, bool NORMED = false, bool ATOMIC = false>
 __global__ __launch_bounds__(512) void stream_kernel(Tokens tk, const bf16_t* __restrict__ w,
-                                                  TO* __restrict__ out, int M, int n_out, int K, int groups, int act = 0) {
+                                                  TO* __restrict__ out, int M, int n_out, int K, int groups, int act = 0,
+                                                  const float* __restrict__ col_scale = nullptr) {
   constexpr int WV = 8, U = 8, NACC = SWIGLU ? 2 : 1;
   extern __shared__ __align__(16) unsigned char stream_smem[];
   const int steps_all = K >> 5;
@@ -500,7 +503,7 @@ __global__ __launch_bounds__(512) void stream_kernel(Tokens tk, const bf16_t* __
         for (int v = 0; v < 4; ++v) {
           const int n = (tile0 + rt) * 16 + 4 * g + v;
           if (n >= n_out) continue;
-          if constexpr (ATOMIC) add_to(dst + n, sum[v]);
+          if constexpr (ATOMIC) add_to(dst + n, col_scale != nullptr ? col_scale[n] * sum[v] : sum[v]);
           else dst[n] = from_float<TO>(sum[v]);
         }
       }
@@ -521,7 +524,7 @@ static Tokens plain_tokens(const void* x) { return Tokens{static_cast<const bf16
 // workgroups: how many may stay per K-slice; the groups are dealt out evenly over them.
 template <int RT, int ROWS, bool SWIGLU, bool NORMED = false, bool ATOMIC = false>
 static int launch_stream(hipStream_t s, const Tokens& tk, const void* w, void* out, int out_dtype, int M, int n_out, int K,
-                         int ksplit, int workgroups) {
+                         int ksplit, int workgroups, const float* col_scale = nullptr) {
   const int groups = static_cast<int>(ceil_div(ceil_div(n_out, 16), RT));
   const size_t smem = stream_smem_bytes(RT, ROWS, SWIGLU, K, ksplit);
   const int rounds = static_cast<int>(ceil_div(groups, workgroups));
@@ -533,7 +536,7 @@ static int launch_stream(hipStream_t s, const Tokens& tk, const void* w, void* o
       set_error("psamd_linear_skinny: " + std::to_string(smem) + " bytes of LDS were refused");
       return -1;
     }
-    kernel<<<grid, block, smem, s>>>(tk, wp, dst, M, n_out, K, groups, g_gate_act);
+    kernel<<<grid, block, smem, s>>>(tk, wp, dst, M, n_out, K, groups, g_gate_act, col_scale);
     return check_launch("psamd_linear_skinny");
   };
   if constexpr (ATOMIC) {
@@ -1017,7 +1020,8 @@ int psamd_normed_supports(int M, int K) { return normed_ok(M, K) ? 1 : 0; }
 // over as many workgroups as fill the chip, and every slice adds its partial sums with float
 // atomics that return nothing. The order of the additions is not fixed: results differ in the
 // last bit from run to run.
-int psamd_linear_skinny_add(void* stream, const void* x, const void* w, float* out, int M, int n_out, int K) {
+int psamd_linear_skinny_add(void* stream, const void* x, const void* w, float* out, int M, int n_out, int K,
+                            const float* col_scale) {
   PSAMD_REQUIRE(M >= 1 && M <= 16, "M must be in [1, 16]");
   PSAMD_REQUIRE(n_out > 0 && K > 0 && K % 8 == 0, "K must be a positive multiple of 8");
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -1025,12 +1029,12 @@ int psamd_linear_skinny_add(void* stream, const void* x, const void* w, float* o
   const int64_t groups = ceil_div(n_out, 16);
   const int wgs = ksplit > 1 ? 512 / ksplit : 0;
   if (M >= 4 && K % 32 == 0 && wgs > 0 && groups >= 2 * wgs && stream_smem_bytes(1, 16, false, K, ksplit) <= 160 * 1024) {
-    if (M <= 8) return launch_stream<1, 8, false, false, true>(s, plain_tokens(x), w, out, kF32, M, n_out, K, ksplit, wgs);
-    return launch_stream<1, 16, false, false, true>(s, plain_tokens(x), w, out, kF32, M, n_out, K, ksplit, wgs);
+    if (M <= 8) return launch_stream<1, 8, false, false, true>(s, plain_tokens(x), w, out, kF32, M, n_out, K, ksplit, wgs, col_scale);
+    return launch_stream<1, 16, false, false, true>(s, plain_tokens(x), w, out, kF32, M, n_out, K, ksplit, wgs, col_scale);
   }
   const dim3 grid(static_cast<unsigned>(groups), static_cast<unsigned>(ksplit)), block(64 * 4);
   skinny_mfma_kernel<1, 1, 4, false, true, float, 8, true><<<grid, block, 0, s>>>(
-      static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), out, M, n_out, K);
+      static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), out, M, n_out, K, 0, col_scale);
   return check_launch("psamd_linear_skinny_add");
 }
 

@@ -14,7 +14,16 @@
 // -limit, limit), act = g * sigmoid(gate_alpha * g) * (u + up_shift), out = down act. There the weight
 // multiplies the expert's input, so it cannot be pulled out of the clamps; with weight_on_output the
 // expert sees x itself and the weight multiplies out (limit = infinity, gate_alpha = 1, up_shift = 0
-// then make the plain SiLU-gated expert).
+// then make the plain SiLU-gated expert). The other kind of expert has no gate: act = max(up h, 0)^2
+// (kExpertSquaredRelu), its first matrix is [F, K].
+//
+// With groups (mode 0): the experts form `groups` equal runs of neighbours, a run's score is the sum of its
+// two largest scores, and only experts of the `keep` best runs (the lower index among equals) can be
+// chosen. The weights are multiplied by `factor`.
+//
+// `out` is float slices [top][tokens][K], or, for a small bfloat16 step, the float residual stream itself
+// (`into_stream`): every pair then adds col_scale[k] * weight * value with float atomics, and nobody adds
+// slices up afterwards (the order of the additions differs from run to run).
 
 #include <algorithm>
 
@@ -25,6 +34,20 @@ namespace psamd {
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
+
+constexpr int kExpertGated = 0, kExpertSquaredRelu = 1;
+constexpr int kMaxRouterGroups = 4 * kWave;
+
+// How a router turns scores into a choice (see above). groups 0: every expert can be chosen.
+struct RouterRule {
+  int mode;
+  int groups;
+  int keep;
+  float factor;
+};
+
+// dst += v at the memory side, nothing returned.
+__device__ __forceinline__ void add_float(float* dst, float v) { (void)unsafeAtomicAdd(dst, v); }
 
 // Dot product of a row of n elements with a float vector in LDS, dealt out over the 64 lanes;
 // every lane returns the whole sum. bfloat16 rows whose length is a multiple of 8 are read in
@@ -66,12 +89,76 @@ __device__ __forceinline__ float wave_dot(const W* __restrict__ row, const float
 
 // ------------------------------------------------------------------ router
 
+// The largest of every lane's (value, index), the lower index among equals, in every lane.
+__device__ __forceinline__ void wave_best(float& best, int& at) {
+#pragma unroll
+  for (int o = kWave / 2; o > 0; o >>= 1) {
+    const float ob = __shfl_xor(best, o, kWave);
+    const int oa = __shfl_xor(at, o, kWave);
+    if (ob > best || (ob == best && oa < at)) {
+      best = ob;
+      at = oa;
+    }
+  }
+}
+
+// Takes the experts outside the best groups out of the choice: their entries of score[] (LDS) become kTaken.
+// Lane l holds the scores of groups l, l + 64, ... (at most kMaxRouterGroups in all).
+__device__ __forceinline__ void keep_best_groups(float* score, int experts, int groups, int keep, int lane) {
+  constexpr int kPer = kMaxRouterGroups / kWave;
+  const float kTaken = -__builtin_inff();
+  const int size = experts / groups;
+  float sum[kPer];
+  bool kept[kPer];
+#pragma unroll
+  for (int i = 0; i < kPer; ++i) {
+    const int grp = lane + i * kWave;
+    kept[i] = false;
+    sum[i] = kTaken;
+    if (grp < groups) {
+      float a = kTaken, b = 0.f;                          // the two largest; a group of one expert has one
+      for (int e = grp * size; e < (grp + 1) * size; ++e) {
+        const float s = score[e];
+        if (s > a) {
+          b = a == kTaken ? 0.f : a;
+          a = s;
+        } else if (e > grp * size + 1 ? s > b : e > grp * size) {
+          b = s;
+        }
+      }
+      sum[i] = a + b;
+    }
+  }
+  for (int j = 0; j < keep; ++j) {
+    float best = kTaken;
+    int at = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < kPer; ++i)
+      if (!kept[i] && sum[i] > best) {                    // ascending groups: the first of equals stays
+        best = sum[i];
+        at = lane + i * kWave;
+      }
+    wave_best(best, at);
+#pragma unroll
+    for (int i = 0; i < kPer; ++i) kept[i] = kept[i] || at == lane + i * kWave;
+  }
+#pragma unroll
+  for (int i = 0; i < kPer; ++i) {
+    const int grp = lane + i * kWave;
+    if (grp < groups && !kept[i])
+      for (int e = grp * size; e < (grp + 1) * size; ++e) score[e] = kTaken;
+  }
+  __builtin_amdgcn_wave_barrier();
+  __threadfence_block();
+}
+
 // The router's choice for one token by one wave: score[] (LDS, `experts` entries: sigmoid(z) in mode
 // 0, z in mode 1) -> chosen / weight [top], largest first, the lower index among equals; taken
 // entries are overwritten. Mode 1 then turns the chosen z into their softmax.
-__device__ __forceinline__ void pick_top(float* score, int experts, int top, int mode, int32_t* __restrict__ chosen,
+__device__ __forceinline__ void pick_top(float* score, int experts, int top, RouterRule rule, int32_t* __restrict__ chosen,
                                          float* __restrict__ weight, int lane) {
   const float kTaken = -__builtin_inff();
+  if (rule.groups > 0) keep_best_groups(score, experts, rule.groups, rule.keep, lane);
   for (int j = 0; j < top; ++j) {
     float best = kTaken;
     int at = 0x7fffffff;
@@ -82,28 +169,20 @@ __device__ __forceinline__ void pick_top(float* score, int experts, int top, int
         at = e;
       }
     }
-#pragma unroll
-    for (int o = kWave / 2; o > 0; o >>= 1) {
-      const float ob = __shfl_xor(best, o, kWave);
-      const int oa = __shfl_xor(at, o, kWave);
-      if (ob > best || (ob == best && oa < at)) {
-        best = ob;
-        at = oa;
-      }
-    }
+    wave_best(best, at);
     if (lane == 0) {
       chosen[j] = at;
-      weight[j] = best;
+      weight[j] = rule.mode == 0 ? rule.factor * best : best;
       if (at != 0x7fffffff) score[at] = kTaken;
     }
     __builtin_amdgcn_wave_barrier();
     __threadfence_block();
   }
-  if (mode == 1 && lane == 0) {
+  if (rule.mode == 1 && lane == 0) {
     const float m = weight[0];                           // the largest comes first
     float sum = 0.f;
     for (int j = 0; j < top; ++j) sum += expf(weight[j] - m);
-    for (int j = 0; j < top; ++j) weight[j] = expf(weight[j] - m) / sum;
+    for (int j = 0; j < top; ++j) weight[j] = rule.factor * (expf(weight[j] - m) / sum);
   }
 }
 
@@ -118,7 +197,8 @@ __device__ __forceinline__ float router_score(float z, const float* __restrict__
 template <typename A>
 __global__ __launch_bounds__(256) void moe_route_kernel(const A* __restrict__ x, const float* __restrict__ w_router,
                                                         int32_t* __restrict__ chosen, float* __restrict__ weight,
-                                                        int K, int experts, int top, const float* __restrict__ bias, int mode) {
+                                                        int K, int experts, int top, const float* __restrict__ bias,
+                                                        RouterRule rule) {
   extern __shared__ __align__(16) float route_smem[];    // xs[K], score[experts]
   float* xs = route_smem;
   float* score = route_smem + K;
@@ -128,27 +208,27 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const A* __restrict__ x,
   __syncthreads();
   for (int e = wave; e < experts; e += 4) {
     const float z = wave_dot<float>(w_router + static_cast<int64_t>(e) * K, xs, K, lane);
-    if (lane == 0) score[e] = router_score(z, bias, e, mode);
+    if (lane == 0) score[e] = router_score(z, bias, e, rule.mode);
   }
   __syncthreads();
   if (wave != 0) return;
-  pick_top(score, experts, top, mode, chosen + t * top, weight + t * top, lane);
+  pick_top(score, experts, top, rule, chosen + t * top, weight + t * top, lane);
 }
 
 // The same choice from logits a product has already written (z[t, :] float). One wave per token,
 // four tokens per block.
 __global__ __launch_bounds__(256) void moe_topk_kernel(const float* __restrict__ z, int32_t* __restrict__ chosen,
                                                        float* __restrict__ weight, int64_t tokens, int experts, int top,
-                                                       const float* __restrict__ bias, int mode) {
+                                                       const float* __restrict__ bias, RouterRule rule) {
   extern __shared__ __align__(16) float topk_smem[];     // score[4][experts]
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x >> 6;
   const int64_t t = static_cast<int64_t>(blockIdx.x) * 4 + wave;
   if (t >= tokens) return;
   float* score = topk_smem + wave * experts;
-  for (int e = lane; e < experts; e += kWave) score[e] = router_score(z[t * experts + e], bias, e, mode);
+  for (int e = lane; e < experts; e += kWave) score[e] = router_score(z[t * experts + e], bias, e, rule.mode);
   __builtin_amdgcn_wave_barrier();
   __threadfence_block();
-  pick_top(score, experts, top, mode, chosen + t * top, weight + t * top, lane);
+  pick_top(score, experts, top, rule, chosen + t * top, weight + t * top, lane);
 }
 
 // ------------------------------------------------------------------ experts, pair by pair
@@ -162,7 +242,7 @@ template <typename A>
 __global__ __launch_bounds__(256) void moe_gate_up_rows_kernel(
     const A* __restrict__ x, const int32_t* __restrict__ chosen, const float* __restrict__ weight,
     const A* __restrict__ w_gate_up, A* __restrict__ act, int K, int F, int experts, int top, float gate_alpha,
-    float limit, float up_shift, int weight_on_output) {
+    float limit, float up_shift, int weight_on_output, int kind) {
   extern __shared__ __align__(16) float rows_smem[];     // h[K]
   const int64_t pair = blockIdx.x;
   const int64_t t = pair / top;
@@ -171,12 +251,17 @@ __global__ __launch_bounds__(256) void moe_gate_up_rows_kernel(
   const float wgt = weight_on_output ? 1.f : weight[pair];
   for (int i = threadIdx.x; i < K; i += blockDim.x) rows_smem[i] = wgt * to_float<A>(x[t * K + i]);
   __syncthreads();
-  const A* we = w_gate_up + static_cast<int64_t>(e) * 2 * F * K;
+  const A* we = w_gate_up + static_cast<int64_t>(e) * (kind == kExpertGated ? 2 : 1) * F * K;
 #pragma unroll
   for (int r = 0; r < kRowsPerWave; ++r) {
     const int f = static_cast<int>(blockIdx.y) * kRowsPerBlock + wave * kRowsPerWave + r;
     if (f >= F) break;
     float g = wave_dot<A>(we + static_cast<int64_t>(f) * K, rows_smem, K, lane);
+    if (kind == kExpertSquaredRelu) {
+      g = fmaxf(g, 0.f);
+      if (lane == 0) act[pair * F + f] = from_float<A>(g * g);
+      continue;
+    }
     float u = wave_dot<A>(we + static_cast<int64_t>(F + f) * K, rows_smem, K, lane);
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
@@ -188,7 +273,8 @@ __global__ __launch_bounds__(256) void moe_gate_up_rows_kernel(
 template <typename A>
 __global__ __launch_bounds__(256) void moe_down_rows_kernel(
     const A* __restrict__ act, const int32_t* __restrict__ chosen, const A* __restrict__ w_down,
-    float* __restrict__ out, int64_t tokens, int K, int F, int experts, int top, const float* __restrict__ out_weight) {
+    float* __restrict__ out, int64_t tokens, int K, int F, int experts, int top, const float* __restrict__ out_weight,
+    int into_stream, const float* __restrict__ col_scale) {
   extern __shared__ __align__(16) float rows_smem[];     // act[F]
   const int64_t pair = blockIdx.x;
   const int64_t t = pair / top;
@@ -198,13 +284,16 @@ __global__ __launch_bounds__(256) void moe_down_rows_kernel(
   for (int i = threadIdx.x; i < F; i += blockDim.x) rows_smem[i] = to_float<A>(act[pair * F + i]);
   __syncthreads();
   const A* we = w_down + static_cast<int64_t>(e) * K * F;
-  float* o = out + (static_cast<int64_t>(j) * tokens + t) * K;
+  float* o = out + (into_stream ? t : static_cast<int64_t>(j) * tokens + t) * K;
 #pragma unroll
   for (int r = 0; r < kRowsPerWave; ++r) {
     const int k = static_cast<int>(blockIdx.y) * kRowsPerBlock + wave * kRowsPerWave + r;
     if (k >= K) break;
     const float v = wave_dot<A>(we + static_cast<int64_t>(k) * F, rows_smem, F, lane);
-    if (lane == 0) o[k] = out_weight != nullptr ? out_weight[pair] * v : v;
+    if (lane != 0) continue;
+    const float y = out_weight != nullptr ? out_weight[pair] * v : v;
+    if (into_stream) add_float(o + k, col_scale != nullptr ? col_scale[k] * y : y);
+    else o[k] = y;
   }
 }
 
@@ -268,15 +357,15 @@ __global__ __launch_bounds__(1024) void moe_topk_group_kernel(const float* __res
                                                               int tile_rows, int max_tiles, int32_t* __restrict__ sorted,
                                                               int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_first,
                                                               int32_t* __restrict__ tile_count, const float* __restrict__ bias,
-                                                              int mode) {
+                                                              RouterRule rule) {
   extern __shared__ int32_t group_smem[];      // as above, then score[16][experts]
   float* score = reinterpret_cast<float*>(group_smem + 4 * experts + 1) + (threadIdx.x >> 6) * experts;
   const int lane = threadIdx.x & (kWave - 1);
   for (int t = threadIdx.x >> 6; t < tokens; t += 16) {
-    for (int e = lane; e < experts; e += kWave) score[e] = router_score(z[static_cast<int64_t>(t) * experts + e], bias, e, mode);
+    for (int e = lane; e < experts; e += kWave) score[e] = router_score(z[static_cast<int64_t>(t) * experts + e], bias, e, rule.mode);
     __builtin_amdgcn_wave_barrier();
     __threadfence_block();
-    pick_top(score, experts, top, mode, chosen + t * top, weight + t * top, lane);
+    pick_top(score, experts, top, rule, chosen + t * top, weight + t * top, lane);
   }
   __threadfence_block();
   __syncthreads();                             // the workgroup's own writes of `chosen` are read below
@@ -296,15 +385,19 @@ constexpr int kGroupLD = kGroupBK + 8;         // LDS row stride of the staged p
 // rows that belong to them) and multiplies them with all MT tiles of pairs. The next round's
 // rows of both operands are asked for before the current round is multiplied (registers, then
 // the other of two LDS buffers), so one barrier per round is all the waves wait for.
-//   GATED: out_act[pair][n] = act(gate, up) in bfloat16, N = F columns, w = [E][2N][K].
-//   else:  out_f32[(pair % top) * tokens + pair / top][n] = sum, N = hidden columns, w = [E][N][K],
-//          rows of `a` are indexed by pair.
-template <int MT, int RT, bool GATED>
+//   kFormGated:       out_act[pair][n] = act(gate, up) in bfloat16, N = F columns, w = [E][2N][K].
+//   kFormSquaredRelu: out_act[pair][n] = max(sum, 0)^2 in bfloat16, N = F columns, w = [E][N][K].
+//   kFormDown: out_f32[(pair % top) * tokens + pair / top][n] = sum, N = hidden columns, w = [E][N][K],
+//              rows of `a` are indexed by pair; into_stream: out_f32[pair / top][n] += col_scale[n] * sum.
+constexpr int kFormDown = 0, kFormGated = 1, kFormSquaredRelu = 2;
+template <int MT, int RT, int FORM>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const bf16_t* __restrict__ a, const float* __restrict__ pair_weight, const bf16_t* __restrict__ w,
     const int32_t* __restrict__ sorted, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_first,
     const int32_t* __restrict__ tile_count, bf16_t* __restrict__ out_act, float* __restrict__ out_f32, int64_t tokens,
-    int K, int N, int top, float gate_alpha, float limit, float up_shift) {
+    int K, int N, int top, float gate_alpha, float limit, float up_shift, int into_stream,
+    const float* __restrict__ col_scale) {
+  constexpr bool GATED = FORM == kFormGated;
   constexpr int ROWS = MT * 16;
   constexpr int PIECES = ROWS * (kGroupBK / 8);              // 16-byte pieces of a round's pairs
   constexpr int PPT = (PIECES + 255) / 256;                  // pieces per thread
@@ -340,7 +433,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const int idx = static_cast<int>(threadIdx.x) + p * 256;
     const int row = min(idx, PIECES - 1) / (kGroupBK / 8), c = min(idx, PIECES - 1) % (kGroupBK / 8);
     const int pair = pair_s[row];
-    src[p] = (pair >= 0 && idx < PIECES) ? a + static_cast<int64_t>(GATED ? pair / top : pair) * K + 8 * c : nullptr;
+    src[p] = (pair >= 0 && idx < PIECES) ? a + static_cast<int64_t>(FORM != kFormDown ? pair / top : pair) * K + 8 * c : nullptr;
   }
   uint4 areg[PPT];
   bf16x8 wa[KK][RT], wb[KK][RT];
@@ -421,11 +514,16 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
       const int nc = n0 + rt * 16 + 4 * g;
-      if (GATED) {
+      if (FORM != kFormDown) {
         bf16_t* o = out_act + static_cast<int64_t>(pair) * N + nc;
         bf16_t res[4];
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
+          if (!GATED) {
+            const float p = fmaxf(pw * acc_g[rt][mt][v], 0.f);
+            res[v] = float_to_bf16(p * p);
+            continue;
+          }
           const float gg = fminf(pw * acc_g[rt][mt][v], limit);
           const float uu = fminf(fmaxf(pw * acc_u[rt][mt][v], -limit), limit);
           res[v] = float_to_bf16(gg / (1.f + __expf(-gate_alpha * gg)) * (uu + up_shift));
@@ -437,6 +535,11 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
           for (int v = 0; v < 4; ++v)
             if (nc + v < N) o[v] = res[v];
         }
+      } else if (into_stream) {
+        float* o = out_f32 + static_cast<int64_t>(pair / top) * N + nc;
+#pragma unroll
+        for (int v = 0; v < 4; ++v)
+          if (nc + v < N) add_float(o + v, (col_scale != nullptr ? col_scale[nc + v] : 1.f) * (pw * acc_g[rt][mt][v]));
       } else {
         float* o = out_f32 + (static_cast<int64_t>(pair % top) * tokens + pair / top) * N + nc;
         if (nc + 3 < N && (N & 3) == 0) {
@@ -451,40 +554,69 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
   }
 }
 
-template <int MT, int RT>
-static int launch_grouped(hipStream_t s, const void* x, const float* weight, const void* w_gate_up, const void* w_down,
-                          void* act, float* out, const int32_t* ints, int max_tiles, int64_t tokens, int K, int F, int top,
-                          float gate_alpha, float limit, float up_shift, int weight_on_output) {
-  const int64_t pairs = tokens * top;
+// What the experts' two products have in common.
+struct ExpertCall {
+  const void* x;
+  const int32_t* chosen;
+  const float* weight;
+  const void* w_in;                    // [E, 2F, K] (gated) or [E, F, K]
+  const void* w_down;                  // [E, K, F]
+  void* act;
+  float* out;
+  int64_t tokens;
+  int K, F, experts, top, kind;
+  float gate_alpha, limit, up_shift;
+  int weight_on_output, into_stream;
+  const float* col_scale;
+};
+
+template <int MT, int RT, int FORM>
+static void run_grouped(hipStream_t s, const ExpertCall& c, const int32_t* ints, int max_tiles) {
   const int32_t* sorted = ints;
-  const int32_t* t_e = ints + pairs;
+  const int32_t* t_e = ints + c.tokens * c.top;
   const int32_t* t_f = t_e + max_tiles;
   const int32_t* t_c = t_f + max_tiles;
-  moe_grouped_kernel<MT, RT, true><<<dim3(static_cast<unsigned>(ceil_div(F, 64 * RT)), static_cast<unsigned>(max_tiles)), dim3(256), 0, s>>>(
-      static_cast<const bf16_t*>(x), weight_on_output ? nullptr : weight, static_cast<const bf16_t*>(w_gate_up), sorted, t_e, t_f, t_c,
-      static_cast<bf16_t*>(act), nullptr, tokens, K, F, top, gate_alpha, limit, up_shift);
-  if (check_launch("psamd_moe_experts_grouped (gate/up)")) return 1;
-  moe_grouped_kernel<MT, RT, false><<<dim3(static_cast<unsigned>(ceil_div(K, 64 * RT)), static_cast<unsigned>(max_tiles)), dim3(256), 0, s>>>(
-      static_cast<const bf16_t*>(act), weight_on_output ? weight : nullptr, static_cast<const bf16_t*>(w_down), sorted, t_e, t_f, t_c, nullptr, out,
-      tokens, F, K, top, 0.f, 0.f, 0.f);
+  constexpr bool down = FORM == kFormDown;
+  const int N = down ? c.K : c.F, K = down ? c.F : c.K;
+  const dim3 grid(static_cast<unsigned>(ceil_div(N, 64 * RT)), static_cast<unsigned>(max_tiles));
+  moe_grouped_kernel<MT, RT, FORM><<<grid, dim3(256), 0, s>>>(
+      static_cast<const bf16_t*>(down ? c.act : c.x), (c.weight_on_output != 0) == down ? c.weight : nullptr,
+      static_cast<const bf16_t*>(down ? c.w_down : c.w_in), sorted, t_e, t_f, t_c, down ? nullptr : static_cast<bf16_t*>(c.act),
+      down ? c.out : nullptr, c.tokens, K, N, c.top, c.gate_alpha, c.limit, c.up_shift, c.into_stream, c.col_scale);
+}
+
+template <int MT, int RT>
+static int launch_grouped(hipStream_t s, const ExpertCall& c, const int32_t* ints, int max_tiles) {
+  if (c.kind == kExpertGated) run_grouped<MT, RT, kFormGated>(s, c, ints, max_tiles);
+  else run_grouped<MT, RT, kFormSquaredRelu>(s, c, ints, max_tiles);
+  if (check_launch("psamd_moe_experts_grouped (in)")) return 1;
+  run_grouped<MT, RT, kFormDown>(s, c, ints, max_tiles);
   return check_launch("psamd_moe_experts_grouped (down)");
 }
 
 template <typename A>
-static int launch_experts_rows(hipStream_t s, const void* x, const int32_t* chosen, const float* weight,
-                               const void* w_gate_up, const void* w_down, void* act, float* out, int64_t tokens, int K,
-                               int F, int experts, int top, float gate_alpha, float limit, float up_shift,
-                               int weight_on_output) {
-  const unsigned pairs = static_cast<unsigned>(tokens * top);
-  moe_gate_up_rows_kernel<A><<<dim3(pairs, static_cast<unsigned>(ceil_div(F, kRowsPerBlock))), dim3(256),
-                               sizeof(float) * K, s>>>(
-      static_cast<const A*>(x), chosen, weight, static_cast<const A*>(w_gate_up), static_cast<A*>(act), K, F, experts, top,
-      gate_alpha, limit, up_shift, weight_on_output);
-  if (check_launch("psamd_moe_experts_rows (gate/up)")) return 1;
-  moe_down_rows_kernel<A><<<dim3(pairs, static_cast<unsigned>(ceil_div(K, kRowsPerBlock))), dim3(256), sizeof(float) * F,
-                            s>>>(static_cast<const A*>(act), chosen, static_cast<const A*>(w_down), out, tokens, K, F,
-                                 experts, top, weight_on_output ? weight : nullptr);
+static int launch_experts_rows(hipStream_t s, const ExpertCall& c) {
+  const unsigned pairs = static_cast<unsigned>(c.tokens * c.top);
+  moe_gate_up_rows_kernel<A><<<dim3(pairs, static_cast<unsigned>(ceil_div(c.F, kRowsPerBlock))), dim3(256),
+                               sizeof(float) * c.K, s>>>(
+      static_cast<const A*>(c.x), c.chosen, c.weight, static_cast<const A*>(c.w_in), static_cast<A*>(c.act), c.K, c.F,
+      c.experts, c.top, c.gate_alpha, c.limit, c.up_shift, c.weight_on_output, c.kind);
+  if (check_launch("psamd_moe_experts_rows (in)")) return 1;
+  moe_down_rows_kernel<A><<<dim3(pairs, static_cast<unsigned>(ceil_div(c.K, kRowsPerBlock))), dim3(256),
+                            sizeof(float) * c.F, s>>>(
+      static_cast<const A*>(c.act), c.chosen, static_cast<const A*>(c.w_down), c.out, c.tokens, c.K, c.F, c.experts, c.top,
+      c.weight_on_output ? c.weight : nullptr, c.into_stream, c.col_scale);
   return check_launch("psamd_moe_experts_rows (down)");
+}
+
+// The rule as the entry points take it, checked on the host.
+static const char* bad_rule(int mode, int groups, int keep, int experts, int top) {
+  if (mode != 0 && mode != 1) return "router mode 0 (sigmoid scores) or 1 (softmax over the chosen)";
+  if (groups == 0) return nullptr;
+  if (mode != 0) return "groups of experts go with sigmoid scores";
+  if (groups < 1 || groups > kMaxRouterGroups || experts % groups != 0) return "the experts must form at most 256 equal groups";
+  if (keep < 1 || keep > groups || top > keep * (experts / groups)) return "the kept groups hold fewer experts than are chosen";
+  return nullptr;
 }
 
 // out[t, :] *= sigmoid(x[t] . w): one number per token on the output of a branch every token takes.
@@ -511,9 +643,11 @@ int psamd_moe_grouped_tile_rows(int64_t pairs, int experts);
 int psamd_moe_grouped_max_tiles(int64_t pairs, int experts);
 
 int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_router, int32_t* chosen, float* weight,
-                    int64_t tokens, int K, int experts, int top, const float* bias, int mode) {
-  PSAMD_REQUIRE(mode == 0 || mode == 1, "router mode 0 (sigmoid scores) or 1 (softmax over the chosen)");
+                    int64_t tokens, int K, int experts, int top, const float* bias, int mode,
+                    int groups, int keep, float factor) {
   PSAMD_REQUIRE(tokens >= 0 && K > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
+  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
+  const RouterRule rule{mode, groups, keep, factor};
   PSAMD_REQUIRE(sizeof(float) * (static_cast<size_t>(K) + experts) <= 64 * 1024, "row and scores do not fit in LDS");
   PSAMD_REQUIRE(tokens <= 2147483647LL, "too many tokens for one launch");
   if (tokens == 0) return 0;
@@ -522,10 +656,10 @@ int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_rou
   const dim3 grid(static_cast<unsigned>(tokens));
   if (x_dtype == kBF16) {
     moe_route_kernel<bf16_t><<<grid, dim3(256), smem, s>>>(static_cast<const bf16_t*>(x), w_router, chosen, weight, K,
-                                                          experts, top, bias, mode);
+                                                          experts, top, bias, rule);
   } else if (x_dtype == kF32) {
     moe_route_kernel<float><<<grid, dim3(256), smem, s>>>(static_cast<const float*>(x), w_router, chosen, weight, K,
-                                                         experts, top, bias, mode);
+                                                         experts, top, bias, rule);
   } else {
     return fail("psamd_moe_route: x must be float32 or bfloat16");
   }
@@ -533,21 +667,25 @@ int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_rou
 }
 
 int psamd_moe_topk(void* stream, const float* logits, int32_t* chosen, float* weight, int64_t tokens, int experts,
-                   int top, const float* bias, int mode) {
-  PSAMD_REQUIRE(mode == 0 || mode == 1, "router mode 0 (sigmoid scores) or 1 (softmax over the chosen)");
+                   int top, const float* bias, int mode,
+                   int groups, int keep, float factor) {
   PSAMD_REQUIRE(tokens >= 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
+  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
+  const RouterRule rule{mode, groups, keep, factor};
   PSAMD_REQUIRE(sizeof(float) * 4 * static_cast<size_t>(experts) <= 64 * 1024, "scores do not fit in LDS");
   PSAMD_REQUIRE(ceil_div(tokens, 4) <= 2147483647LL, "too many tokens for one launch");
   if (tokens == 0) return 0;
   moe_topk_kernel<<<dim3(static_cast<unsigned>(ceil_div(tokens, 4))), dim3(256), sizeof(float) * 4 * experts,
-                    static_cast<hipStream_t>(stream)>>>(logits, chosen, weight, tokens, experts, top, bias, mode);
+                    static_cast<hipStream_t>(stream)>>>(logits, chosen, weight, tokens, experts, top, bias, rule);
   return check_launch("psamd_moe_topk");
 }
 
 int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, float* weight, int32_t* ints, int64_t tokens,
-                         int experts, int top, const float* bias, int mode) {
-  PSAMD_REQUIRE(mode == 0 || mode == 1, "router mode 0 (sigmoid scores) or 1 (softmax over the chosen)");
+                         int experts, int top, const float* bias, int mode,
+                         int groups, int keep, float factor) {
   PSAMD_REQUIRE(tokens >= 1 && tokens <= 64 && experts > 0 && experts <= 1024 && top >= 1 && top <= experts, "bad sizes");
+  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
+  const RouterRule rule{mode, groups, keep, factor};
   PSAMD_REQUIRE(ints != nullptr, "the grouping needs its integer scratch");
   const int64_t pairs = tokens * top;
   const int rows = psamd_moe_grouped_tile_rows(pairs, experts);
@@ -555,25 +693,24 @@ int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, flo
   moe_topk_group_kernel<<<dim3(1), dim3(1024), sizeof(int32_t) * (4 * experts + 1) + sizeof(float) * 16 * experts,
                           static_cast<hipStream_t>(stream)>>>(logits, chosen, weight, static_cast<int>(tokens), experts, top, rows,
                                                               max_tiles, ints, ints + pairs, ints + pairs + max_tiles,
-                                                              ints + pairs + 2 * max_tiles, bias, mode);
+                                                              ints + pairs + 2 * max_tiles, bias, rule);
   return check_launch("psamd_moe_topk_group");
 }
 
 int psamd_moe_experts_rows(void* stream, const void* x, const int32_t* chosen, const float* weight,
-                           const void* w_gate_up, const void* w_down, void* act, float* out, int dtype,
+                           const void* w_in, const void* w_down, void* act, float* out, int dtype,
                            int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
-                           float up_shift, int weight_on_output) {
+                           float up_shift, int weight_on_output, int kind, int into_stream, const float* col_scale) {
   PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
+  PSAMD_REQUIRE(kind == kExpertGated || kind == kExpertSquaredRelu, "experts are gated (0) or squared ReLU without a gate (1)");
   PSAMD_REQUIRE(sizeof(float) * static_cast<size_t>(std::max(K, F)) <= 64 * 1024, "a row does not fit in LDS");
   PSAMD_REQUIRE(tokens * top <= 2147483647LL && ceil_div(std::max(K, F), kRowsPerBlock) <= 65535, "too large for one launch");
   if (tokens == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (dtype == kBF16)
-    return launch_experts_rows<bf16_t>(s, x, chosen, weight, w_gate_up, w_down, act, out, tokens, K, F, experts, top,
-                                       gate_alpha, limit, up_shift, weight_on_output);
-  if (dtype == kF32)
-    return launch_experts_rows<float>(s, x, chosen, weight, w_gate_up, w_down, act, out, tokens, K, F, experts, top,
-                                      gate_alpha, limit, up_shift, weight_on_output);
+  const ExpertCall c{x, chosen, weight, w_in, w_down, act, out, tokens, K, F, experts, top, kind,
+                     gate_alpha, limit, up_shift, weight_on_output, into_stream, col_scale};
+  if (dtype == kBF16) return launch_experts_rows<bf16_t>(s, c);
+  if (dtype == kF32) return launch_experts_rows<float>(s, c);
   return fail("psamd_moe_experts_rows: dtype must be float32 or bfloat16");
 }
 
@@ -592,9 +729,11 @@ int psamd_moe_grouped_max_tiles(int64_t pairs, int experts) {
 }
 
 int psamd_moe_experts_grouped(void* stream, const void* x, const int32_t* chosen, const float* weight,
-                              const void* w_gate_up, const void* w_down, void* act, float* out, int32_t* ints,
+                              const void* w_in, const void* w_down, void* act, float* out, int32_t* ints,
                               int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
-                              float up_shift, int grouped_already, int weight_on_output) {
+                              float up_shift, int grouped_already, int weight_on_output, int kind, int into_stream,
+                              const float* col_scale) {
+  PSAMD_REQUIRE(kind == kExpertGated || kind == kExpertSquaredRelu, "experts are gated (0) or squared ReLU without a gate (1)");
   PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
   PSAMD_REQUIRE(K % 8 == 0 && F % 8 == 0, "K and F must be multiples of 8");
   PSAMD_REQUIRE(experts <= 4096 && tokens * top <= (1 << 24), "too many experts or pairs");
@@ -611,14 +750,11 @@ int psamd_moe_experts_grouped(void* stream, const void* x, const int32_t* chosen
         ints + pairs + 2 * max_tiles);
     if (check_launch("psamd_moe_experts_grouped (grouping)")) return 1;
   }
-  if (rows == 128)
-    return launch_grouped<8, 2>(s, x, weight, w_gate_up, w_down, act, out, ints, max_tiles, tokens, K, F, top, gate_alpha,
-                                limit, up_shift, weight_on_output);
-  if (rows == 64)
-    return launch_grouped<4, 2>(s, x, weight, w_gate_up, w_down, act, out, ints, max_tiles, tokens, K, F, top, gate_alpha,
-                                limit, up_shift, weight_on_output);
-  return launch_grouped<1, 1>(s, x, weight, w_gate_up, w_down, act, out, ints, max_tiles, tokens, K, F, top, gate_alpha, limit,
-                              up_shift, weight_on_output);
+  const ExpertCall c{x, chosen, weight, w_in, w_down, act, out, tokens, K, F, experts, top, kind,
+                     gate_alpha, limit, up_shift, weight_on_output, into_stream, col_scale};
+  if (rows == 128) return launch_grouped<8, 2>(s, c, ints, max_tiles);
+  if (rows == 64) return launch_grouped<4, 2>(s, c, ints, max_tiles);
+  return launch_grouped<1, 1>(s, c, ints, max_tiles);
 }
 
 int psamd_row_gate(void* stream, float* out, const void* x, int act_dtype, const float* w, int64_t tokens, int out_hidden,

@@ -19,7 +19,7 @@ from typing import Any, Sequence
 import torch
 
 from prefixserve_amd.build import ensure_kernels
-from prefixserve_amd.parts.base import NormedRows
+from prefixserve_amd.parts.base import NormedRows, ScaledDelta
 
 _F32, _BF16 = 0, 1
 _vp, _i32, _i64, _f32 = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_float
@@ -45,7 +45,7 @@ logger = logging.getLogger(__name__)
 
 _SIGNATURES = {
     "psamd_embed": [_vp, _vp, _vp, _i32, _vp, _i64, _i32, _i32],
-    "psamd_add_rmsnorm": [_vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _i32, _f32, _vp, _i32, _i64, _i32],
+    "psamd_add_rmsnorm": [_vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _vp, _i32, _f32, _vp, _i32, _i64, _i32],
     "psamd_swiglu": [_vp, _vp, _vp, _i32, _i64, _i32, _i32],
     "psamd_rope_kv_append": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _vp, _vp, _vp, _vp],
     "psamd_linear": [_vp, _vp, _i32, _vp, _i32, _vp, _i32, _i64, _i32, _i32],
@@ -54,7 +54,7 @@ _SIGNATURES = {
     "psamd_linear_skinny_ksplit": [_i32, _i32, _i32],
     "psamd_qkv_rope_append": [_vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _vp, _vp],
     "psamd_normed_supports": [_i32, _i32],
-    "psamd_linear_skinny_add": [_vp, _vp, _vp, _vp, _i32, _i32, _i32],
+    "psamd_linear_skinny_add": [_vp, _vp, _vp, _vp, _i32, _i32, _i32, _vp],
     "psamd_linear_normed": [_vp, _vp, _vp, _vp, _i32, _f32, _vp, _vp, _i32, _i32, _i32, _i32, _i32],
     "psamd_qkv_rope_append_normed": [_vp, _vp, _vp, _i32, _f32, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _vp, _vp],
     "psamd_attention_generic": [_vp, _vp, _i32, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32,
@@ -78,20 +78,24 @@ _SIGNATURES = {
     "psamd_to_activation": [_vp, _vp, _vp, _i32, _i64],
     "psamd_rope_norm_kv_append": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _vp, _vp, _i32, _f32, _vp, _vp],
     "psamd_qk_prepare_kv_append": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _vp, _vp, _i32, _f32, _vp, _vp, _vp, _i32, _vp, _vp, _i32],
-    "psamd_residual_add": [_vp, _vp, _vp, _i32, _i32, _i64, _i64, _i32],
+    "psamd_residual_add": [_vp, _vp, _vp, _i32, _i32, _i64, _i64, _i32, _vp, _vp],
     "psamd_stream_affine": [_vp, _vp, _i64, _i32, _f32, _vp],
     "psamd_concat_to_activation": [_vp, _vp, _vp, _vp, _i32, _i64, _i32],
-    "psamd_heads_linear": [_vp, _vp, _i32, _i64, _i32, _vp, _i32, _vp, _i32, _i64, _i32, _i64, _i32, _i32, _i32],
-    "psamd_latent_kv_append": [_vp, _vp, _i64, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _vp, _f32, _vp, _vp],
+    "psamd_heads_linear": [_vp, _vp, _i32, _i64, _i32, _vp, _i32, _vp, _i32, _i64, _i32, _i64, _i32, _i32, _i32, _vp, _i64, _i32],
+    "psamd_latent_kv_append": [_vp, _vp, _i64, _vp, _i64, _i32, _vp, _vp, _vp, _i64, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _i32,
+                               _vp, _vp, _vp, _f32, _vp, _vp],
+    "psamd_latent_query": [_vp, _vp, _i64, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _vp],
     "psamd_causal_conv": [_vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i64, _i32, _i32],
     "psamd_gated_scan": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _i32,
                          _vp, _i32, _i32, _vp, _i32, _vp, _i32, _i32, _i32],
-    "psamd_moe_route": [_vp, _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _vp, _i32],
-    "psamd_moe_topk": [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32],
+    "psamd_moe_route": [_vp, _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
+    "psamd_moe_topk": [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
     "psamd_moe_grouped_max_tiles": [_i64, _i32],
-    "psamd_moe_experts_grouped": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32, _i32],
-    "psamd_moe_topk_group": [_vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32],
-    "psamd_moe_experts_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32],
+    "psamd_moe_experts_grouped": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32, _i32,
+                                  _i32, _i32, _vp],
+    "psamd_moe_topk_group": [_vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
+    "psamd_moe_experts_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32,
+                               _i32, _i32, _vp],
     "psamd_row_gate": [_vp, _vp, _vp, _i32, _vp, _i64, _i32, _i32],
     "psamd_layernorm_step": [_vp, _vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _f32, _vp, _vp, _f32, _vp, _i32, _i64, _i32],
     "psamd_add_sinusoid": [_vp, _vp, _vp, _vp, _i64, _i32],
@@ -119,6 +123,8 @@ _SIGNATURES = {
     "psamd_attention_masked": [_vp, _vp, _i32, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32,
                                _vp, _vp, _vp, _i32, _vp],
 }
+
+EXPERT_KINDS = {"gated": 0, "squared_relu": 1}
 
 ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3}
 
@@ -282,23 +288,34 @@ class HipOps:
         self._need(delta.shape == (t, h) and delta.dtype == out_dtype, "delta must match the output")
         return delta.data_ptr(), _code(delta.dtype), 1, 0
 
+    def _scaled(self, delta, h: int) -> tuple:
+        """(the delta itself, pointer to its factors per column or None)."""
+        if not isinstance(delta, ScaledDelta):
+            return delta, None
+        self._need(delta.scale.dtype == torch.float32 and delta.scale.numel() == h and delta.scale.is_contiguous(),
+                   "a delta's factors per column are float32 [H]")
+        return delta.delta, delta.scale.data_ptr()
+
     def add_rmsnorm(self, residual, delta, weight, eps: float, out) -> None:
+        """residual += delta (a ``ScaledDelta``: times its factors per column), out = weight * rmsnorm(residual)."""
         t, h = residual.shape
+        delta, scale = self._scaled(delta, h)
         self._need(residual.dtype == torch.float32 and residual.is_contiguous(), "add_rmsnorm: residual must be float32")
         self._need(out.shape == (t, h) and out.is_contiguous(), "add_rmsnorm: bad output shape")
         self._need(weight.numel() == h, "add_rmsnorm: weight size")
         dptr, dcode, slices, stride = self._delta_args(delta, t, h, out.dtype)
-        self._ok(self.lib.psamd_add_rmsnorm(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride, None,
+        self._ok(self.lib.psamd_add_rmsnorm(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride, scale, None,
                                             weight.data_ptr(), _code(weight.dtype), eps, out.data_ptr(),
                                             _code(out.dtype), t, h))
 
     def add_rmsnorm_rows(self, residual, delta, rows, weight, eps: float, out) -> None:
         t, h = residual.shape
+        delta, scale = self._scaled(delta, h)
         s = rows.numel()
         self._need(residual.dtype == torch.float32 and rows.dtype == torch.int32, "add_rmsnorm_rows: dtypes")
         self._need(out.shape == (s, h) and out.is_contiguous(), "add_rmsnorm_rows: bad output shape")
         dptr, dcode, slices, stride = self._delta_args(delta, t, h, out.dtype)
-        self._ok(self.lib.psamd_add_rmsnorm(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride,
+        self._ok(self.lib.psamd_add_rmsnorm(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride, scale,
                                             rows.data_ptr(), weight.data_ptr(), _code(weight.dtype), eps,
                                             out.data_ptr(), _code(out.dtype), s, h))
 
@@ -328,14 +345,17 @@ class HipOps:
         self._ok(self.lib.psamd_swiglu(self._stream(), gate_up.data_ptr(), out.data_ptr(), _code(out.dtype), t, inter,
                                        GATE_ACTIVATIONS[activation]))
 
-    def residual_add(self, residual, delta) -> None:
+    def residual_add(self, residual, delta, row=None) -> None:
         """residual (float32 [T, H]) += delta: [T, H] in any kernel dtype, or [S, T, H] float32 slices
-        (added in ascending order). For an arrangement that adds a sub-layer's output without a
-        norm behind the sum."""
+        (added in ascending order), or a ``ScaledDelta`` of either. ``row`` (float32 [H]) is added to every
+        row as well. For an arrangement that adds a sub-layer's output without a norm behind the sum."""
         t, h = residual.shape
+        delta, scale = self._scaled(delta, h)
+        if row is not None:
+            self._need(row.dtype == torch.float32 and row.numel() == h and row.is_contiguous(), "residual_add: the row is float32 [H]")
         self._need(residual.dtype == torch.float32 and residual.is_contiguous(), "residual_add: the stream is float32")
         dptr, dcode, slices, stride = self._delta_args(delta, t, h, delta.dtype)
-        self._ok(self.lib.psamd_residual_add(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride, t, h))
+        self._ok(self.lib.psamd_residual_add(self._stream(), residual.data_ptr(), dptr, dcode, slices, stride, t, h, scale, _ptr(row)))
 
     def stream_affine(self, x, factor: float = 1.0, row=None) -> None:
         """x (float32 [T, H]) <- x * factor + row (float32 [H] or None), in place."""
@@ -353,10 +373,12 @@ class HipOps:
         self._ok(self.lib.psamd_concat_to_activation(self._stream(), a.data_ptr(), b.data_ptr(), out.data_ptr(),
                                                      _code(out.dtype), t, h))
 
-    def heads_linear(self, x, x_offset: int, x_head: int, w, out, out_offset: int, out_head: int) -> None:
+    def heads_linear(self, x, x_offset: int, x_head: int, w, out, out_offset: int, out_head: int, gate=None,
+                     gate_offset: int = 0, gate_head: int = 0) -> None:
         """One small product per head: out[t, out_offset + h * out_head + n] = sum_k x[t, x_offset + h * x_head + k]
         * w[h, n, k] for w [H, N, K]; x and out are 2-d and contiguous, their heads lie inside their
-        rows. One dtype for x, w and out; float accumulation."""
+        rows. One dtype for x, w and out; float accumulation. ``gate`` (rows of the same dtype): every result is
+        multiplied by sigmoid(gate[t, gate_offset + h * gate_head + n])."""
         heads, n, k = w.shape
         m = x.shape[0]
         self._need(x.dim() == 2 and out.dim() == 2 and x.is_contiguous() and out.is_contiguous() and w.is_contiguous()
@@ -365,35 +387,73 @@ class HipOps:
         self._need(x_offset >= 0 and x_offset + (heads - 1) * x_head + k <= x.shape[1]
                    and out_offset >= 0 and out_offset + (heads - 1) * out_head + n <= out.shape[1], "heads_linear: heads outside their rows")
         size = x.element_size()
+        gptr, grow = None, 0
+        if gate is not None:
+            self._need(gate.dtype == x.dtype and gate.dim() == 2 and gate.shape[0] == m and gate.is_contiguous() and gate_offset >= 0
+                       and gate_offset + (heads - 1) * gate_head + n <= gate.shape[1], "heads_linear: the gate's columns")
+            gptr, grow = gate.data_ptr() + gate_offset * size, gate.shape[1]
         self._ok(self.lib.psamd_heads_linear(
             self._stream(), x.data_ptr() + x_offset * size, _code(x.dtype), x.shape[1], x_head, w.data_ptr(), _code(w.dtype),
-            out.data_ptr() + out_offset * size, _code(out.dtype), out.shape[1], out_head, m, heads, n, k))
+            out.data_ptr() + out_offset * size, _code(out.dtype), out.shape[1], out_head, m, heads, n, k, gptr, grow, gate_head))
 
-    def latent_kv_append(self, rows, q_lat, hq: int, dim: int, rot: int, rank: int, slots: int, positions, table,
-                         norm_weight, eps: float, kv, write_slot) -> None:
-        """Latent attention between its input product and the attention: ``rows`` [T, hq (dim + rot) + rank + rot]
-        holds the heads' queries and the token's compressed vector with the shared key part. The
-        compressed vector is normalized (weight, eps), the key part and every head's last ``rot``
-        query dimensions are rotated pair by pair (neighbours; ``table`` [pos, rot/2, 2]); the page
-        receives key and value, ``q_lat`` [T, hq * slots] every head's rotated part at [rank, rank + rot)
-        and zeros behind it."""
-        t = rows.shape[0]
-        self._need(rows.is_contiguous() and q_lat.is_contiguous() and q_lat.dtype == rows.dtype
-                   and rows.shape[1] >= hq * (dim + rot) + rank + rot and q_lat.shape == (t, hq * slots), "latent_kv_append: shapes")
-        self._need(positions.dtype == torch.int32 and positions.numel() == t, "latent_kv_append: positions")
-        self._need(norm_weight.dtype == torch.float32 and norm_weight.numel() == rank and norm_weight.is_contiguous(),
-                   "latent_kv_append: the norm's weight is float32 [rank]")
+    def _latent_table(self, table, rot: int, positions, t: int) -> None:
+        self._need(positions.dtype == torch.int32 and positions.numel() == t, "latent attention: positions")
         if rot:
             self._need(table is not None and table.dtype == torch.float32 and table.shape[1:] == (rot // 2, 2)
-                       and table.is_contiguous() and table.shape[0] >= 1, "latent_kv_append: table must be float32 [positions, rot/2, 2]")
+                       and table.is_contiguous() and table.shape[0] >= 1, "latent attention: the table must be float32 [positions, rot/2, 2]")
+
+    def latent_kv_append(self, rows, q_lat, hq: int, dim: int, rot: int, rank: int, slots: int, positions, table,
+                         norm_weight, eps: float, kv, write_slot, halves: bool = False, low_col: int | None = None,
+                         q_latent=None) -> None:
+        """Latent attention between its input product and the attention. ``rows`` [T, >= ...] holds the
+        token's compressed vector with the shared key part from column ``low_col`` on (None: behind hq
+        heads of dim + rot query dimensions). The compressed vector is normalized (weight, eps), the key
+        part is rotated pair by pair (partners neighbours, or rot/2 apart with ``halves``; ``table`` [pos,
+        rot/2, 2]) and the page receives key and value. ``q_lat`` [T, hq * slots] (None: the queries do
+        not lie in ``rows``): every head's last ``rot`` query dimensions go rotated to [rank, rank + rot), zeros
+        behind them. ``q_latent`` = (columns, weight, out): the queries' own latent, ``rows``' first columns,
+        normed like the compressed vector into ``out`` [T, columns]."""
+        t = rows.shape[0]
+        low = hq * (dim + rot) if low_col is None else int(low_col)
+        self._need(rows.is_contiguous() and 0 <= low and low + rank + rot <= rows.shape[1], "latent_kv_append: shapes")
+        self._latent_table(table, rot, positions, t)
+        self._need(norm_weight.dtype == torch.float32 and norm_weight.numel() == rank and norm_weight.is_contiguous(),
+                   "latent_kv_append: the norm's weight is float32 [rank]")
+        size = rows.element_size()
+        qptr = None
+        if q_lat is not None:
+            self._need(hq * (dim + rot) <= rows.shape[1] and q_lat.is_contiguous() and q_lat.dtype == rows.dtype
+                       and q_lat.shape == (t, hq * slots), "latent_kv_append: queries")
+            qptr = rows.data_ptr()
+        cptr = cw = cout = None
+        c_rank = 0
+        if q_latent is not None:
+            c_rank, weight, out = q_latent
+            self._need(0 < c_rank <= rows.shape[1] and weight.dtype == torch.float32 and weight.numel() == c_rank and weight.is_contiguous()
+                       and out.shape == (t, c_rank) and out.dtype == rows.dtype and out.is_contiguous(), "latent_kv_append: the queries' latent")
+            cptr, cw, cout = rows.data_ptr(), weight.data_ptr(), out.data_ptr()
         if kv is not None:
             self._need(kv.dtype == rows.dtype and kv.shape[1:] == (2, 1, 16 * slots) and kv.is_contiguous(),
                        "latent_kv_append: cache must be [blocks, 2, 1, 16 * slots] in the activation dtype")
             self._need(write_slot.dtype == torch.int32 and write_slot.numel() == t, "latent_kv_append: write slots")
-        self._ok(self.lib.psamd_latent_kv_append(self._stream(), rows.data_ptr(), rows.shape[1], q_lat.data_ptr(), _code(rows.dtype),
-                                                 t, hq, dim, rot, rank, slots, positions.data_ptr(), _ptr(table),
-                                                 norm_weight.data_ptr(), float(eps), _ptr(kv),
-                                                 None if kv is None else write_slot.data_ptr()))
+        self._ok(self.lib.psamd_latent_kv_append(
+            self._stream(), rows.data_ptr() + low * size, rows.shape[1], cptr, rows.shape[1], c_rank, cw, cout, qptr, rows.shape[1],
+            _ptr(q_lat), _code(rows.dtype), t, hq, dim, rot, rank, slots, int(halves), positions.data_ptr(), _ptr(table),
+            norm_weight.data_ptr(), float(eps), _ptr(kv), None if kv is None else write_slot.data_ptr()))
+
+    def latent_query(self, q, w_fold, q_lat, hq: int, dim: int, rot: int, rank: int, slots: int, positions, table,
+                     halves: bool = False) -> None:
+        """q_lat[t, h] = [w_fold[h] . q[t, h, :dim] | rotated q[t, h, dim:] | zeros] for q [T, hq (dim + rot)] and
+        w_fold [hq, rank, dim]: the queries as the attention in the compressed space reads them."""
+        t = q.shape[0]
+        self._need(q.is_contiguous() and q.shape[1] == hq * (dim + rot) and q_lat.is_contiguous() and q_lat.dtype == q.dtype
+                   and q_lat.shape == (t, hq * slots), "latent_query: shapes")
+        self._need(w_fold.shape == (hq, rank, dim) and w_fold.dtype == q.dtype and w_fold.is_contiguous(), "latent_query: w_fold")
+        self._latent_table(table, rot, positions, t)
+        if dim == 0:
+            q_lat.view(t, hq, slots)[:, :, :rank].zero_()
+        self._ok(self.lib.psamd_latent_query(self._stream(), q.data_ptr(), q.shape[1], w_fold.data_ptr(), q_lat.data_ptr(), _code(q.dtype),
+                                             t, hq, dim, rot, rank, slots, int(halves), positions.data_ptr(), _ptr(table)))
 
     def _state_args(self, state, ctx, width: int, taps: int) -> tuple:
         self._need(state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous()
@@ -590,22 +650,29 @@ class HipOps:
         self._ok(self.lib.psamd_linear(self._stream(), x.data_ptr(), _code(x.dtype), w.data_ptr(), _code(w.dtype),
                                        out.data_ptr(), _code(out.dtype), m, n, k))
 
-    def linear_to_residual(self, x, w, name: str, residual: torch.Tensor | None = None) -> torch.Tensor | None:
+    def linear_to_residual(self, x, w, name: str, residual: torch.Tensor | None = None,
+                           col_scale: torch.Tensor | None = None) -> torch.Tensor | None:
         """x @ w^T for a consumer that adds it to the residual stream (the fused add+norm).
         Returns [T, N] in the activation dtype or, for a small bfloat16 step whose product has
         few output columns, [S, T, N] float32 partial sums of a K-split, which the consumer adds
         up: splitting K over workgroups is what lets such a product use the whole chip. With the
         stream itself given as ``residual`` (float32 [T, N]), a step small enough to run without
-        norm kernels adds the product into it here, K-slice by K-slice, and returns None."""
+        norm kernels adds the product into it here, K-slice by K-slice, and returns None.
+        ``col_scale`` (float32 [N]): what is added into ``residual`` here is multiplied by it column by
+        column; what is returned is not (the caller hands it on as a ``ScaledDelta``)."""
         m, k = x.shape
         n = w.shape[0]
         if (residual is not None and 0 < m and x.dtype == torch.bfloat16 and k % 8 == 0 and residual.shape == (m, n)
                 and self.fuses_norm(m, n, x.dtype)):
             self._need(residual.dtype == torch.float32 and residual.is_contiguous(), "the residual stream is float32")
             self._need(w.shape[1] == k and x.is_contiguous() and w.is_contiguous(), "linear_to_residual: operands")
-            self._ok(self.lib.psamd_linear_skinny_add(self._stream(), x.data_ptr(), w.data_ptr(), residual.data_ptr(), m, n, k))
+            if col_scale is not None:
+                self._need(col_scale.dtype == torch.float32 and col_scale.numel() == n and col_scale.is_contiguous(),
+                           "linear_to_residual: the factors per column are float32 [N]")
+            self._ok(self.lib.psamd_linear_skinny_add(self._stream(), x.data_ptr(), w.data_ptr(), residual.data_ptr(), m, n, k,
+                                                      _ptr(col_scale)))
             return None
-        if (residual is not None and m >= self.LIBRARY_ADD_MIN_ROWS and x.dtype == torch.bfloat16 and k % 8 == 0
+        if (residual is not None and col_scale is None and m >= self.LIBRARY_ADD_MIN_ROWS and x.dtype == torch.bfloat16 and k % 8 == 0
                 and residual.shape == (m, n) and residual.dtype == torch.float32 and self._direct_library):
             # A large step: the library's product adds into the float32 stream itself (out = x w^T + out),
             # so the sum is not rounded to bfloat16 on its way there and the norm that follows reads the
@@ -674,7 +741,8 @@ class HipOps:
 
     # ------------------------------------------------------------------ experts
 
-    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode: int = 0) -> None:
+    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode: int = 0, groups: int = 0,
+                  keep: int = 0, factor: float = 1.0) -> None:
         """chosen[t, :], weight[t, :] = the experts with the largest sigmoid(x[t] . w_router[e]) and
         those scores, largest first, the lower index among equals; scores in 32-bit. With the router
         also given in the activation dtype (``w_router_act``), a step of more than
@@ -683,7 +751,9 @@ class HipOps:
         the whole router once per token with one workgroup (8 tokens of a 32 x 2,048 router: 94 us
         against 5 + 4 for product and choice), so the bound is 0 and it serves callers without that copy.
         ``bias`` (float32 [E]) is added to the logits; ``mode`` 1: the largest logits are chosen and the
-        weights are the softmax over the chosen logits alone."""
+        weights are the softmax over the chosen logits alone. ``groups`` > 0: the experts form that many equal
+        runs of neighbours, a run's score is the sum of its two largest scores, and only experts of the ``keep`` best
+        runs can be chosen. The weights are multiplied by ``factor``."""
         if bias is not None:
             self._need(bias.dtype == torch.float32 and bias.numel() == w_router.shape[0] and bias.is_contiguous(),
                        "moe_route: the bias is float32 [E]")
@@ -701,11 +771,11 @@ class HipOps:
                 # A small step: the workgroup that chooses also sorts the pairs for the experts' kernels.
                 ints = self._group_ints(t, top, e)
                 self._ok(self.lib.psamd_moe_topk_group(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
-                                                       ints.data_ptr(), t, e, top, _ptr(bias), int(mode)))
+                                                       ints.data_ptr(), t, e, top, _ptr(bias), int(mode), int(groups), int(keep), float(factor)))
                 self._grouped_for = (chosen.data_ptr(), t, top, e)
                 return
             self._ok(self.lib.psamd_moe_topk(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(), t, e, top,
-                                             _ptr(bias), int(mode)))
+                                             _ptr(bias), int(mode), int(groups), int(keep), float(factor)))
             return
         self._grouped_for = None
         self._need(x.is_contiguous() and w_router.dtype == torch.float32 and w_router.is_contiguous()
@@ -714,7 +784,8 @@ class HipOps:
                    and weight.shape == (t, top) and chosen.is_contiguous() and weight.is_contiguous() and 1 <= top <= e,
                    "moe_route: outputs must be int32 and float32 [T, top]")
         self._ok(self.lib.psamd_moe_route(self._stream(), x.data_ptr(), _code(x.dtype), w_router.data_ptr(),
-                                          chosen.data_ptr(), weight.data_ptr(), t, k, e, top, _ptr(bias), int(mode)))
+                                          chosen.data_ptr(), weight.data_ptr(), t, k, e, top, _ptr(bias), int(mode), int(groups), int(keep),
+                                          float(factor)))
 
     def _groups_pairs(self, dtype: torch.dtype, t: int, k: int) -> bool:
         """Whether a step of ``t`` tokens of width ``k`` runs its experts grouped by expert."""
@@ -724,37 +795,51 @@ class HipOps:
         tiles = int(self.lib.psamd_moe_grouped_max_tiles(t * top, e))
         return self.ws.get("moe.group", (t * top + 3 * tiles,), torch.int32)
 
-    def moe_experts(self, x, chosen, weight, w_gate_up, w_down, act, out, gate_alpha: float, limit: float,
-                    up_shift: float, weight_on_output: bool = False) -> None:
+    def moe_experts(self, x, chosen, weight, w_in, w_down, act, out, gate_alpha: float, limit: float,
+                    up_shift: float, weight_on_output: bool = False, kind: str = "gated", residual=None, col_scale=None) -> None:
         """out[j, t] = down_e(act_e(weight[t, j] * x[t])) for e = chosen[t, j], as float32 slices [top, T, K];
         ``act`` [T * top, F] is scratch in the activation dtype. ``weight_on_output``: out[j, t] =
-        weight[t, j] * down_e(act_e(x[t])) instead."""
+        weight[t, j] * down_e(act_e(x[t])) instead. ``kind`` "gated": ``w_in`` is [E, 2F, K], gate rows in front of up
+        rows; "squared_relu": [E, F, K], act_e(h) = max(w_in h, 0)^2. ``residual`` (float32 [T, K], instead of
+        ``out``, which is then None; bfloat16 only): every pair adds its output, times ``col_scale`` (float32 [K]) if
+        given, into it with float atomics."""
         t, k = x.shape
         top = chosen.shape[1]
-        e, f2, _ = w_gate_up.shape
-        f = f2 // 2
-        self._need(w_gate_up.shape == (e, 2 * f, k) and w_down.shape == (e, k, f) and w_gate_up.is_contiguous()
-                   and w_down.is_contiguous() and w_gate_up.dtype == x.dtype and w_down.dtype == x.dtype,
-                   "moe_experts: weights must be [E, 2F, K] and [E, K, F] in the activation dtype")
+        e, _, f = w_down.shape
+        rows = 2 * f if kind == "gated" else f
+        self._need(w_in.shape == (e, rows, k) and w_down.shape == (e, k, f) and w_in.is_contiguous()
+                   and w_down.is_contiguous() and w_in.dtype == x.dtype and w_down.dtype == x.dtype,
+                   "moe_experts: weights must be [E, 2F (gated) or F, K] and [E, K, F] in the activation dtype")
         self._need(x.is_contiguous() and chosen.shape == (t, top) and weight.shape == (t, top) and chosen.dtype == torch.int32
                    and weight.dtype == torch.float32 and chosen.is_contiguous() and weight.is_contiguous(),
                    "moe_experts: the router's outputs")
         self._need(act.shape == (t * top, f) and act.dtype == x.dtype and act.is_contiguous(), "moe_experts: act scratch")
-        self._need(out.shape == (top, t, k) and out.dtype == torch.float32 and out.is_contiguous(), "moe_experts: output slices")
+        into = residual is not None
+        if into:
+            self._need(out is None and residual.dtype == torch.float32 and residual.shape == (t, k) and residual.is_contiguous()
+                       and x.dtype == torch.bfloat16, "moe_experts: the residual stream is float32 [T, K], in a bfloat16 step")
+            if col_scale is not None:
+                self._need(col_scale.dtype == torch.float32 and col_scale.numel() == k and col_scale.is_contiguous(),
+                           "moe_experts: the factors per column are float32 [K]")
+            out = residual
+        else:
+            self._need(col_scale is None and out.shape == (top, t, k) and out.dtype == torch.float32 and out.is_contiguous(),
+                       "moe_experts: output slices")
+        tail = (int(weight_on_output), EXPERT_KINDS[kind], int(into), _ptr(col_scale))
         if self._groups_pairs(x.dtype, t, k) and f % 8 == 0:
             # Sorted by expert and run in tiles on the matrix cores: an expert is read once per tile of pairs.
             ints = self._group_ints(t, top, e)
             done = int(getattr(self, "_grouped_for", None) == (chosen.data_ptr(), t, top, e))   # the router's kernel sorted them
             self._grouped_for = None
             self._ok(self.lib.psamd_moe_experts_grouped(self._stream(), x.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
-                                                        w_gate_up.data_ptr(), w_down.data_ptr(), act.data_ptr(),
+                                                        w_in.data_ptr(), w_down.data_ptr(), act.data_ptr(),
                                                         out.data_ptr(), ints.data_ptr(), t, k, f, e, top, float(gate_alpha),
-                                                        float(limit), float(up_shift), done, int(weight_on_output)))
+                                                        float(limit), float(up_shift), done, *tail))
             return
         self._ok(self.lib.psamd_moe_experts_rows(self._stream(), x.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
-                                                 w_gate_up.data_ptr(), w_down.data_ptr(), act.data_ptr(), out.data_ptr(),
+                                                 w_in.data_ptr(), w_down.data_ptr(), act.data_ptr(), out.data_ptr(),
                                                  _code(x.dtype), t, k, f, e, top, float(gate_alpha), float(limit),
-                                                 float(up_shift), int(weight_on_output)))
+                                                 float(up_shift), *tail))
 
     def row_gate(self, out, x, w) -> None:
         """out[t, :] *= sigmoid(x[t] . w): float32 out [T, N], x [T, K] in a kernel dtype, w float32 [K]."""

@@ -5,3 +5,4 @@ from . import gokolix  # noqa: F401
 from . import larupel  # noqa: F401
 from . import llama  # noqa: F401
 from . import radivik  # noqa: F401
+from . import zurolorn  # noqa: F401

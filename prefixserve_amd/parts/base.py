@@ -120,6 +120,17 @@ class NormedRows:
 
 
 @dataclass
+class ScaledDelta:
+    """A sub-layer's output that is still to be multiplied, column by column, by ``scale`` (float32
+    [hidden]) when it is added to the stream: a block hands it on in place of the output itself, and the
+    kernels that add to the stream (``ops.add_rmsnorm``, ``ops.add_rmsnorm_rows``, ``ops.residual_add``)
+    take it. ``delta`` is in one of the forms ``Mixer.forward`` may return, except None."""
+
+    delta: torch.Tensor
+    scale: torch.Tensor
+
+
+@dataclass
 class WeightedDeltas:
     """What a sub-layer made of several hands to a block that says it takes such (``ctx.takes_weighted_deltas``): the
     sum over ``parts`` of scale * delta, each delta in one of the forms ``Mixer.forward`` may return, to be formed
@@ -218,6 +229,11 @@ class Mixer(Part):
         tokens, say), by a name of the mixer's choosing: the run's ``LayerCache.aux[name]``."""
         return {}
 
+    # True: where ``forward`` adds its output into ``ctx.residual`` itself, it multiplies it by
+    # ``ctx.residual_scale`` (float32 [hidden]) first when that is not None. A block with a learned
+    # factor per column lets only such a sub-layer add into the stream; from others it takes the output.
+    takes_residual_scale = False
+
     # Where in a slot's row this mixer's state begins. 0 when the mixer is the only owner of the
     # run's state; a container (a block with state of its own, a mixer made of several) lays its
     # parts' states side by side and sets this before the first step.
@@ -256,6 +272,10 @@ class Transform(Part):
     tensor's rows belong to (all tokens in order for the stream, ``ctx.logit_rows`` for logits),
     for a transform that depends on the position (``ctx.positions[rows]``)."""
 
+    # A transform of the stream may offer ``add_pending(t, pending, ctx)``: what the last sub-layer left
+    # to be added and then the transform itself, in one go.
+    add_pending = None
+
     def apply(self, t: torch.Tensor, ctx: "StepContext", rows: torch.Tensor | None) -> None:
         raise NotImplementedError
 
@@ -264,6 +284,7 @@ class FeedForward(Part):
     """Per-position transformation (dense or experts)."""
 
     takes_normed_rows = False       # as for Mixer
+    takes_residual_scale = False    # as for Mixer
 
     def forward(self, x: torch.Tensor, ctx: "StepContext") -> torch.Tensor | None:
         """x [T, hidden] -> what is to be added to the residual, as for ``Mixer.forward``."""

@@ -2,14 +2,31 @@
 
 from __future__ import annotations
 
-from typing import TYPE_CHECKING, Any
+from typing import TYPE_CHECKING, Any, Mapping
 
 import torch
 
-from .base import FeedForward, Mixer, Norm, Part, register_block
+from .base import FeedForward, Mixer, Norm, Part, Runtime, ScaledDelta, WeightWant, register_block
 
 if TYPE_CHECKING:
     from prefixserve_amd.engine.batch import StepContext
+
+
+class ColumnScale(Part):
+    """A learned factor per coordinate of the stream (float32 [hidden]) on a sub-layer's output."""
+
+    def __init__(self, hidden_size: int, name: str) -> None:
+        self.hidden_size, self.name = int(hidden_size), name
+
+    def weights(self) -> dict[str, WeightWant]:
+        return {self.name: WeightWant((self.hidden_size,), "norm")}
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
+        super().bind(tensors, rt)
+        self.scale = tensors[self.name].to(device=rt.device, dtype=torch.float32).contiguous()
+
+    def weight_bytes(self) -> int:
+        return 4 * self.hidden_size
 
 
 class PreNormBlock:
@@ -22,14 +39,41 @@ class PreNormBlock:
     their tokens themselves (``takes_normed_rows``), the norm in front of it may hand over the
     rows of the stream instead of running a kernel. An arrangement that needs a sub-layer's
     output itself (to normalize it before it is added, say) sets ``ctx.residual = None`` first:
-    the sub-layers then hand their output back in every step."""
+    the sub-layers then hand their output back in every step.
 
-    def __init__(self, mixer: Mixer, feed_forward: FeedForward, mixer_norm: Norm, feed_forward_norm: Norm) -> None:
+    ``mixer_scale`` / ``feed_forward_scale``: names of learned vectors, one number per coordinate, that
+    multiply the sub-layers' outputs in front of the sums, in 32-bit: in the product that adds into the
+    stream where the sub-layer does (``takes_residual_scale``), else by whoever adds the output
+    (``ScaledDelta``). ``feed_forward`` None: the layer is its mixer alone."""
+
+    def __init__(self, mixer: Mixer, feed_forward: FeedForward | None, mixer_norm: Norm, feed_forward_norm: Norm | None,
+                 mixer_scale: str | None = None, feed_forward_scale: str | None = None) -> None:
+        if (feed_forward is None) != (feed_forward_norm is None) or (feed_forward is None and feed_forward_scale is not None):
+            raise ValueError("a feed-forward comes with its norm, a layer without one has neither norm nor scale for it")
         self.mixer, self.feed_forward = mixer, feed_forward
         self.mixer_norm, self.feed_forward_norm = mixer_norm, feed_forward_norm
+        self.mixer_scale = None if mixer_scale is None else ColumnScale(mixer.hidden_size, mixer_scale)
+        self.feed_forward_scale = None if feed_forward_scale is None else ColumnScale(mixer.hidden_size, feed_forward_scale)
 
     def parts(self) -> list[Part]:
-        return [self.mixer_norm, self.mixer, self.feed_forward_norm, self.feed_forward]
+        every = [self.mixer_norm, self.mixer, self.mixer_scale, self.feed_forward_norm, self.feed_forward, self.feed_forward_scale]
+        return [part for part in every if part is not None]
+
+    @staticmethod
+    def _scaled(part: Any, scale: ColumnScale | None, ctx: "StepContext", *args: Any) -> Any:
+        """``part.forward`` with its output times ``scale``, however it leaves the part."""
+        if scale is None:
+            return part.forward(*args)
+        kept = ctx.residual
+        if part.takes_residual_scale:
+            ctx.residual_scale = scale.scale
+        else:
+            ctx.residual = None
+        try:
+            delta = part.forward(*args)
+        finally:
+            ctx.residual, ctx.residual_scale = kept, None
+        return None if delta is None else ScaledDelta(delta, scale.scale)
 
     def forward(self, residual: torch.Tensor, pending: torch.Tensor | None, ctx: "StepContext", cache: Any,
                 state: torch.Tensor | None, writes_cache: bool) -> torch.Tensor:
@@ -38,12 +82,14 @@ class PreNormBlock:
             x = self.mixer_norm.add_norm(residual, pending, "block.x", lazy=True)
         else:
             x = self.mixer_norm.add_norm(residual, pending, "block.x")
-        mixed = self.mixer.forward(x, ctx, cache, state, writes_cache)
+        mixed = self._scaled(self.mixer, self.mixer_scale, ctx, x, ctx, cache, state, writes_cache)
+        if self.feed_forward is None:
+            return mixed
         if self.feed_forward.takes_normed_rows:
             x = self.feed_forward_norm.add_norm(residual, mixed, "block.x", lazy=True)
         else:
             x = self.feed_forward_norm.add_norm(residual, mixed, "block.x")
-        return self.feed_forward.forward(x, ctx)
+        return self._scaled(self.feed_forward, self.feed_forward_scale, ctx, x, ctx)
 
 
 class PostNormBlock:

@@ -187,6 +187,7 @@ class DecoderModel:
             if s.streams > 1:
                 streams[1:].copy_(residual.unsqueeze(0).expand(s.streams - 1, t, s.hidden_size))
             ctx.residual = residual
+            ctx.residual_scale = None
             ctx.stream_copy = None           # a context may be stepped twice (a graph's eager run, then its capture)
             if self.keeps_embedding_output:
                 ctx.embedding_output = ws.get("embedding.output", (t, s.hidden_size), torch.float32)
@@ -196,13 +197,17 @@ class DecoderModel:
                 if run.before:
                     # A transform reads and writes the stream itself: what the last sub-layer left to
                     # be added goes in first.
-                    if pending is not None:
-                        ops.residual_add(residual, pending)
-                        pending = None
                     ctx.stream_copy = None
                     ctx.pass_index = run.pass_index
-                    for name in run.before:
-                        self.stream_transforms[name].apply(residual, ctx, None)
+                    todo = [self.stream_transforms[name] for name in run.before]
+                    if pending is not None:
+                        if todo[0].add_pending is not None:
+                            todo.pop(0).add_pending(residual, pending, ctx)
+                        else:
+                            ops.residual_add(residual, pending)
+                        pending = None
+                    for tr in todo:
+                        tr.apply(residual, ctx, None)
                 pending = self.blocks[run.layer].forward(streams, pending, ctx, self.caches.get(run.cache),
                                                          self.states.get(i), run.writes_cache)
             if ctx.num_logit_rows == 0:

@@ -1,4 +1,4 @@
-"""Feed-forward as a mixture of experts: a router picks a few small gated feed-forwards per token."""
+"""Feed-forward as a mixture of experts: a router picks a few small feed-forwards per token."""
 
 from __future__ import annotations
 
@@ -13,12 +13,14 @@ if TYPE_CHECKING:
 
 
 class RoutedExperts(FeedForward):
-    """``num_experts`` gated feed-forwards of inner size ``intermediate_size`` without biases, of
+    """``num_experts`` feed-forwards of inner size ``intermediate_size`` without biases, of
     which every token uses ``top_k``.
 
     Router: z = W_r x (+ a bias, ``router_bias``) in 32-bit; the ``top_k`` largest are taken (the
     lower index among equals). ``score`` "sigmoid": the weights are sigmoid(z) as they are, not
-    renormalized; "softmax_of_chosen": the softmax over the chosen z alone.
+    renormalized; "softmax_of_chosen": the softmax over the chosen z alone. ``groups`` = {"count": G, "keep": k}
+    (sigmoid scores): the experts form G equal groups of neighbours, a group's score is the sum of its two
+    largest scores, and only experts of the k best groups can be chosen. ``weight_scale`` multiplies the weights.
 
     ``weight_on`` "input": the weight multiplies the expert's input, the output is the sum over
     the chosen experts of expert(w x), which is not w expert(x) when the expert clamps; "output": the
@@ -26,26 +28,38 @@ class RoutedExperts(FeedForward):
 
     Expert: with g = min(W_gate h, limit) and u = clamp(W_up h, -limit, limit) it is
     W_down (g sigmoid(gate_alpha g) (u + up_shift)); ``limit`` None, ``gate_alpha`` 1 and
-    ``up_shift`` 0 make it W_down (silu(W_gate h) * W_up h).
+    ``up_shift`` 0 make it W_down (silu(W_gate h) * W_up h). ``expert`` "squared_relu": no gate,
+    W_down (max(W_up h, 0))^2; the three constants do not apply.
 
     ``shared`` = {"intermediate_size": F, "gated": bool}: one more SiLU-gated feed-forward that every
     token uses, its output times sigmoid(w . x), one number per token, when ``gated``.
 
     The chosen experts' outputs (and the shared one's) come back as float32 slices ``[top_k (+ 1), T,
     hidden]`` that the norm behind adds up in ascending order, so a token's sum does not depend on
-    what else is in the step. ``names``: "router" ("router_bias"), "gate"/"up"/"down" with ``{e}``
+    what else is in the step; in a bfloat16 step so small that the products add into the residual stream
+    themselves (``ops.fuses_norm``) the experts do so too. ``names``: "router" ("router_bias"), "gate"/"up"/"down" with ``{e}``
     for the expert, "shared_gate"/"shared_up"/"shared_down" ("shared_scale": the [1, hidden] row w)."""
 
+    takes_residual_scale = True
+
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, intermediate_size: int,
-                 names: Mapping[str, str], limit: float | None, gate_alpha: float = 1.702, up_shift: float = 1.0,
+                 names: Mapping[str, str], limit: float | None = None, gate_alpha: float = 1.702, up_shift: float = 1.0,
                  score: str = "sigmoid", renormalize: bool = False, weight_on: str = "input",
-                 router_bias: bool = False, shared: Mapping[str, object] | None = None) -> None:
+                 router_bias: bool = False, shared: Mapping[str, object] | None = None, expert: str = "gated",
+                 groups: Mapping[str, int] | None = None, weight_scale: float = 1.0) -> None:
         if score not in ("sigmoid", "softmax_of_chosen") or renormalize or weight_on not in ("input", "output"):
             raise ValueError("the router kernels score with a sigmoid (scores kept as weights) or with the softmax over the "
                              f"chosen logits, on the experts' input or output; got score={score!r}, "
                              f"renormalize={renormalize}, weight_on={weight_on!r}")
         if not 1 <= top_k <= num_experts:
             raise ValueError(f"top_k {top_k} of {num_experts} experts")
+        if expert not in ("gated", "squared_relu"):
+            raise ValueError(f"experts are gated or squared ReLU without a gate, got {expert!r}")
+        if groups is not None:
+            count, keep = int(groups["count"]), int(groups["keep"])
+            if score != "sigmoid" or not 1 <= count <= 256 or num_experts % count or not 1 <= keep <= count \
+                    or top_k > keep * (num_experts // count):
+                raise ValueError(f"{num_experts} experts in {count} groups of which {keep} are kept, {top_k} chosen, score {score!r}")
         self.hidden_size, self.num_experts, self.top_k = int(hidden_size), int(num_experts), int(top_k)
         self.intermediate_size = int(intermediate_size)
         self.names = dict(names)
@@ -56,8 +70,20 @@ class RoutedExperts(FeedForward):
         self.router_bias = bool(router_bias)
         self.shared_size = None if shared is None else int(shared["intermediate_size"])
         self.shared_gated = shared is not None and bool(shared.get("gated", False))
-        # Whether every call names the newer options, or the older form of the calls serves.
-        self.plain_calls = self.router_mode == 0 and not self.weight_on_output and not self.router_bias
+        self.expert = expert
+        # What the calls name beyond the plain form (sigmoid scores, gated experts, weight on the input).
+        self.route_options: dict[str, object] = {}
+        if self.router_mode or self.router_bias:
+            self.route_options["mode"] = self.router_mode
+        if groups is not None:
+            self.route_options.update(groups=count, keep=keep)
+        if weight_scale != 1.0:
+            self.route_options["factor"] = float(weight_scale)
+        self.expert_options: dict[str, object] = {}
+        if self.weight_on_output:
+            self.expert_options["weight_on_output"] = True
+        if expert != "gated":
+            self.expert_options["kind"] = expert
 
     def weights(self) -> dict[str, WeightWant]:
         h, f, n = self.hidden_size, self.intermediate_size, self.names
@@ -65,7 +91,8 @@ class RoutedExperts(FeedForward):
         if self.router_bias:
             want[n["router_bias"]] = WeightWant((self.num_experts,), "bias")
         for e in range(self.num_experts):
-            want[n["gate"].format(e=e)] = WeightWant((f, h))
+            if self.expert == "gated":
+                want[n["gate"].format(e=e)] = WeightWant((f, h))
             want[n["up"].format(e=e)] = WeightWant((f, h))
             want[n["down"].format(e=e)] = WeightWant((h, f))
         if self.shared_size is not None:
@@ -87,10 +114,10 @@ class RoutedExperts(FeedForward):
         self.b_router = None
         if self.router_bias:
             self.b_router = tensors[n["router_bias"]].to(device=rt.device, dtype=torch.float32).contiguous()
-        # Per expert the rows of gate, then of up: [E, 2F, H]; and down [E, H, F].
-        gate_up = torch.stack([torch.cat([tensors[n["gate"].format(e=e)], tensors[n["up"].format(e=e)]], dim=0)
-                               for e in range(e_n)])
-        self.w_gate_up = rt.ops.prepare_matrix(gate_up, rt)
+        # Per expert the rows of gate (where there is one), then of up: [E, 2F or F, H]; and down [E, H, F].
+        first = ("gate", "up") if self.expert == "gated" else ("up",)
+        self.w_in = rt.ops.prepare_matrix(torch.stack([torch.cat([tensors[n[which].format(e=e)] for which in first], dim=0)
+                                                       for e in range(e_n)]), rt)
         self.w_down = rt.ops.prepare_matrix(torch.stack([tensors[n["down"].format(e=e)] for e in range(e_n)]), rt)
         self.w_shared_gate_up = self.w_shared_down = self.w_shared_scale = None
         if self.shared_size is not None:
@@ -101,27 +128,36 @@ class RoutedExperts(FeedForward):
 
     def weight_bytes(self) -> int:
         """What a decode step of one token reads: the router, ``top_k`` experts and the shared one."""
-        per_expert = (self.w_gate_up.numel() + self.w_down.numel()) // self.num_experts * self.w_down.element_size()
+        per_expert = (self.w_in.numel() + self.w_down.numel()) // self.num_experts * self.w_down.element_size()
         shared = 0
         if self.w_shared_gate_up is not None:
             shared = (self.w_shared_gate_up.numel() + self.w_shared_down.numel()) * self.w_shared_down.element_size()
         return self.w_router.numel() * 4 + self.top_k * per_expert + shared
 
-    def forward(self, x: torch.Tensor, ctx: "StepContext") -> torch.Tensor:
+    def _adds_into_stream(self, t: int, residual: torch.Tensor | None) -> bool:
+        fuses = getattr(self.rt.ops, "fuses_norm", None)
+        return (residual is not None and self.shared_size is None and fuses is not None
+                and fuses(t, self.hidden_size, self.rt.dtype))
+
+    def forward(self, x: torch.Tensor, ctx: "StepContext") -> torch.Tensor | None:
         rt, ops, ws = self.rt, self.rt.ops, self.rt.workspace
         t, k = x.shape[0], self.top_k
         chosen = ws.get("moe.chosen", (t, k), torch.int32)
         weight = ws.get("moe.weight", (t, k), torch.float32)
         act = ws.get("moe.act", (t * k, self.intermediate_size), rt.dtype)
+        if self.b_router is not None:
+            ops.moe_route(x, self.w_router, chosen, weight, self.w_router_act, bias=self.b_router, **self.route_options)
+        else:
+            ops.moe_route(x, self.w_router, chosen, weight, self.w_router_act, **self.route_options)
+        residual = getattr(ctx, "residual", None)
+        if self._adds_into_stream(t, residual):
+            ops.moe_experts(x, chosen, weight, self.w_in, self.w_down, act, None, self.gate_alpha, self.limit, self.up_shift,
+                            residual=residual, col_scale=getattr(ctx, "residual_scale", None), **self.expert_options)
+            return None
         slices = k + (1 if self.shared_size is not None else 0)
         out = ws.get("moe.out", (slices, t, self.hidden_size), torch.float32)
-        if self.plain_calls:
-            ops.moe_route(x, self.w_router, chosen, weight, self.w_router_act)
-            ops.moe_experts(x, chosen, weight, self.w_gate_up, self.w_down, act, out[:k], self.gate_alpha, self.limit, self.up_shift)
-        else:
-            ops.moe_route(x, self.w_router, chosen, weight, self.w_router_act, bias=self.b_router, mode=self.router_mode)
-            ops.moe_experts(x, chosen, weight, self.w_gate_up, self.w_down, act, out[:k], self.gate_alpha, self.limit,
-                            self.up_shift, weight_on_output=self.weight_on_output)
+        ops.moe_experts(x, chosen, weight, self.w_in, self.w_down, act, out[:k], self.gate_alpha, self.limit, self.up_shift,
+                        **self.expert_options)
         if self.shared_size is not None:
             shared_act = ws.get("moe.shared_act", (t, self.shared_size), rt.dtype)
             ops.linear_swiglu(x, self.w_shared_gate_up, shared_act)

@@ -1,5 +1,5 @@
-"""Transforms of the residual stream: a factor behind the token table, and the re-entry into a
-stretch of layers that is passed through several times."""
+"""Transforms of the residual stream: a factor behind the token table, and what happens in front of
+every pass through a stretch of layers that is passed through several times."""
 
 from __future__ import annotations
 
@@ -59,6 +59,33 @@ class StreamReentry(Transform):
         ops.stream_affine(t, 1.0, self.steps[ctx.pass_index])
 
 
+class PassStep(Transform):
+    """In front of every pass through a repeated stretch of layers: x <- x + step[pass], in 32-bit;
+    ``name``: the learned rows [passes, hidden]. What the layer in front left to be added goes in with
+    the same kernel (``add_pending``)."""
+
+    def __init__(self, hidden_size: int, vocab_size: int, passes: int, name: str) -> None:
+        self.hidden_size, self.passes, self.name = int(hidden_size), int(passes), name
+
+    def weights(self) -> dict[str, WeightWant]:
+        return {self.name: WeightWant((self.passes, self.hidden_size), "bias")}
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
+        super().bind(tensors, rt)
+        self.steps = tensors[self.name].to(device=rt.device, dtype=torch.float32).contiguous()
+
+    def _row(self, ctx: "StepContext") -> torch.Tensor:
+        if not 0 <= ctx.pass_index < self.passes:
+            raise ValueError(f"pass {ctx.pass_index} of {self.passes}")
+        return self.steps[ctx.pass_index]
+
+    def apply(self, t: torch.Tensor, ctx: "StepContext", rows: torch.Tensor | None) -> None:
+        self.rt.ops.stream_affine(t, 1.0, self._row(ctx))
+
+    def add_pending(self, t: torch.Tensor, pending: torch.Tensor, ctx: "StepContext") -> None:
+        self.rt.ops.residual_add(t, pending, row=self._row(ctx))
+
+
 class SinusoidalPositions(Transform):
     """t[row, 2i] += sin(p f_i), t[row, 2i + 1] += cos(p f_i) with f_i = base^(-2i / hidden) and p the
     row's position: the fixed table of sines added to the token table's rows. The frequencies are
@@ -82,3 +109,4 @@ class SinusoidalPositions(Transform):
 register_transform("scale", ScaleStream)
 register_transform("sinusoidal_positions", SinusoidalPositions)
 register_transform("reentry", StreamReentry)
+register_transform("pass_step", PassStep)

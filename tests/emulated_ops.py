@@ -13,6 +13,8 @@ import contextlib
 
 import torch
 
+from prefixserve_amd.parts.base import ScaledDelta
+
 PAGE = 16
 
 
@@ -33,22 +35,29 @@ class EmulatedOps:
     def embed(self, ids, table, out) -> None:
         out.copy_(table[ids.long()].float())
 
+    @staticmethod
+    def _whole(delta):
+        """A delta in any of its forms as one float tensor [T, H]."""
+        if isinstance(delta, ScaledDelta):
+            return EmulatedOps._whole(delta.delta) * delta.scale
+        return delta.float().sum(0) if delta.dim() == 3 else delta.float()
+
     def add_rmsnorm(self, residual, delta, weight, eps, out) -> None:
         if delta is not None:
-            residual.add_(delta.float())
+            residual.add_(self._whole(delta))
         x = residual
         out.copy_((weight.float() * x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)).to(out.dtype))
 
     def add_rmsnorm_rows(self, residual, delta, rows, weight, eps, out) -> None:
         x = residual[rows.long()]
         if delta is not None:
-            x = x + (delta[:, rows.long()].float().sum(0) if delta.dim() == 3 else delta[rows.long()].float())
+            x = x + self._whole(delta)[rows.long()]
         out.copy_((weight.float() * x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)).to(out.dtype))
 
     def linear(self, x, w, out) -> None:
         out.copy_((x.float() @ w.float().T).to(out.dtype))
 
-    def linear_to_residual(self, x, w, name, residual=None):
+    def linear_to_residual(self, x, w, name, residual=None, col_scale=None):
         out = self.ws.get(name, (x.shape[0], w.shape[0]), x.dtype)
         self.linear(x, w, out)
         return out
@@ -60,8 +69,10 @@ class EmulatedOps:
                "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh")}[activation]
         out.copy_((act(gu[:, :inter]) * gu[:, inter:]).to(out.dtype))
 
-    def residual_add(self, residual, delta) -> None:
-        residual.add_(delta.float().sum(0) if delta.dim() == 3 else delta.float())
+    def residual_add(self, residual, delta, row=None) -> None:
+        residual.add_(self._whole(delta))
+        if row is not None:
+            residual.add_(row)
 
     def stream_affine(self, x, factor=1.0, row=None) -> None:
         x.mul_(factor)
@@ -71,43 +82,66 @@ class EmulatedOps:
     def concat_to_activation(self, a, b, out) -> None:
         out.copy_(torch.cat([a, b], dim=-1).to(out.dtype))
 
-    def heads_linear(self, x, x_offset, x_head, w, out, out_offset, out_head) -> None:
+    def heads_linear(self, x, x_offset, x_head, w, out, out_offset, out_head, gate=None, gate_offset=0, gate_head=0) -> None:
         heads, n, k = w.shape
         for h in range(heads):
             xs = x[:, x_offset + h * x_head: x_offset + h * x_head + k].float()
-            out[:, out_offset + h * out_head: out_offset + h * out_head + n] = (xs @ w[h].float().T).to(out.dtype)
+            y = xs @ w[h].float().T
+            if gate is not None:
+                y = y * torch.sigmoid(gate[:, gate_offset + h * gate_head: gate_offset + h * gate_head + n].float())
+            out[:, out_offset + h * out_head: out_offset + h * out_head + n] = y.to(out.dtype)
 
-    def latent_kv_append(self, rows, q_lat, hq, dim, rot, rank, slots, positions, table, norm_weight, eps, kv, write_slot) -> None:
+    @staticmethod
+    def _turn(v, table, positions, halves):
+        """v [T, ..., rot] turned by the table's angles; partners rot/2 apart or neighbours."""
+        r = v.shape[-1]
+        cs = table[positions.long()]                       # [t, rot/2, 2]
+        while cs.dim() - 1 < v.dim():
+            cs = cs.unsqueeze(1)
+        one, two = (slice(0, r // 2), slice(r // 2, r)) if halves else (slice(0, r, 2), slice(1, r, 2))
+        a, b = v[..., one], v[..., two]
+        res = torch.empty_like(v)
+        res[..., one] = a * cs[..., 0] - b * cs[..., 1]
+        res[..., two] = b * cs[..., 0] + a * cs[..., 1]
+        return res
+
+    def latent_query(self, q, w_fold, q_lat, hq, dim, rot, rank, slots, positions, table, halves=False) -> None:
+        t = q.shape[0]
+        heads, ql = q.view(t, hq, dim + rot).float(), q_lat.view(t, hq, slots)
+        ql.zero_()
+        for h in range(hq):
+            ql[:, h, :rank] = (heads[:, h, :dim] @ w_fold[h].float().T).to(q_lat.dtype)
+        if rot:
+            ql[:, :, rank: rank + rot] = self._turn(heads[..., dim:], table, positions, halves).to(q_lat.dtype)
+
+    def latent_kv_append(self, rows, q_lat, hq, dim, rot, rank, slots, positions, table, norm_weight, eps, kv, write_slot,
+                         halves=False, low_col=None, q_latent=None) -> None:
         t = rows.shape[0]
-        low = rows[:, hq * (dim + rot):].float()
+        low = rows[:, hq * (dim + rot) if low_col is None else low_col:].float()
+        if q_latent is not None:
+            n, weight, out = q_latent
+            cq = rows[:, :n].float()
+            out.copy_((cq * torch.rsqrt((cq * cq).mean(-1, keepdim=True) + eps) * weight).to(out.dtype))
         c = low[:, :rank]
         c = c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * norm_weight
-
-        def turn(v):                                       # [..., rot], neighbours paired
-            cs = table[positions.long()]                   # [t, rot/2, 2]
-            while cs.dim() - 1 < v.dim():
-                cs = cs.unsqueeze(1)
-            a, b = v[..., 0::2], v[..., 1::2]
-            res = torch.empty_like(v)
-            res[..., 0::2] = a * cs[..., 0] - b * cs[..., 1]
-            res[..., 1::2] = b * cs[..., 0] + a * cs[..., 1]
-            return res
 
         key = torch.zeros((t, slots))
         key[:, :rank] = c
         if rot:
-            key[:, rank: rank + rot] = turn(low[:, rank: rank + rot])
+            key[:, rank: rank + rot] = self._turn(low[:, rank: rank + rot], table, positions, halves)
         val = torch.zeros((t, slots))
         val[:, :rank] = c
         if kv is not None:
             page, off = (write_slot // PAGE).long(), (write_slot % PAGE).long()
             kv[:, 0].view(kv.shape[0], 1, PAGE, slots)[page, 0, off, :] = key.to(kv.dtype)
             kv[:, 1].view(kv.shape[0], 1, slots, PAGE)[page, 0, :, off] = val.to(kv.dtype)
+        if q_lat is None:
+            return
         q = rows[:, : hq * (dim + rot)].view(t, hq, dim + rot).float()
         ql = q_lat.view(t, hq, slots)
         ql[:, :, rank:] = 0
         if rot:
-            ql[:, :, rank: rank + rot] = turn(q[:, :, dim:]).to(q_lat.dtype)
+            ql[:, :, rank: rank + rot] = self._turn(q[:, :, dim:], table, positions, halves).to(q_lat.dtype)
 
     def causal_conv(self, rows, col, bias, conv_w, conv_b, u, state, ctx) -> None:
         width, taps = conv_w.shape
@@ -210,27 +244,36 @@ class EmulatedOps:
             vals = raw_keys if values_from_keys else qkv[:, (hq + hkv) * d:].view(t, hkv, d)
             kv[:, 1].view(kv.shape[0], hkv, d, PAGE)[page, :, :, off] = vals
 
-    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode=0) -> None:
+    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode=0, groups=0, keep=0, factor=1.0) -> None:
         z = x.float() @ w_router.float().T
         if bias is not None:
             z = z + bias
         s = torch.sigmoid(z) if mode == 0 else z
+        if groups:
+            per = s.view(s.shape[0], groups, -1)
+            sums = per.topk(min(2, per.shape[2]), dim=-1).values.sum(-1)
+            best = torch.argsort(-sums, dim=-1, stable=True)[:, :keep]
+            allowed = torch.zeros_like(sums, dtype=torch.bool).scatter_(1, best, True)
+            s = per.masked_fill(~allowed[:, :, None], float("-inf")).reshape(s.shape)
         order = torch.argsort(-s, dim=-1, stable=True)[:, : chosen.shape[1]]
         chosen.copy_(order.to(torch.int32))
         picked = torch.gather(s, 1, order)
-        weight.copy_(picked if mode == 0 else torch.softmax(picked, dim=-1))
+        weight.copy_(factor * (picked if mode == 0 else torch.softmax(picked, dim=-1)))
 
-    def moe_experts(self, x, chosen, weight, w_gate_up, w_down, act, out, gate_alpha, limit, up_shift,
-                    weight_on_output=False) -> None:
+    def moe_experts(self, x, chosen, weight, w_in, w_down, act, out, gate_alpha, limit, up_shift,
+                    weight_on_output=False, kind="gated", residual=None, col_scale=None) -> None:
         t, k = chosen.shape
-        f = w_gate_up.shape[1] // 2
+        f = w_down.shape[2]
         for i in range(t):
             for j in range(k):
                 e = int(chosen[i, j])
                 h = x[i].float() * (1.0 if weight_on_output else weight[i, j])
-                gu = w_gate_up[e].float() @ h
-                g, u = gu[:f].clamp(max=limit), gu[f:].clamp(-limit, limit)
-                y = (g * torch.sigmoid(gate_alpha * g) * (u + up_shift)).to(act.dtype)
+                gu = w_in[e].float() @ h
+                if kind == "gated":
+                    g, u = gu[:f].clamp(max=limit), gu[f:].clamp(-limit, limit)
+                    y = (g * torch.sigmoid(gate_alpha * g) * (u + up_shift)).to(act.dtype)
+                else:
+                    y = gu.clamp(min=0.0).square().to(act.dtype)
                 act[i * k + j] = y
                 out[j, i] = (w_down[e].float() @ y.float()) * (weight[i, j] if weight_on_output else 1.0)
 
