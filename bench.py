@@ -195,9 +195,46 @@ def fubelorn_pair(size: dict, layers: int, vocab: int) -> tuple[dict, dict]:
     return fubelorn, llama
 
 
+# Zurolorn at sizes that resemble real layers, beside the two designs that share its parts and Llama: a Gokolix whose layers
+# are all latent attention with the same sizes (its feed-forward is dense, of the inner size a token passes through here),
+# a Radivik of equal width with experts of the same sizes (gated, so half as many more weights per expert), and the Llama
+# decoder of equal size. Three layers, the second one passed through twice: four layer runs of alternating mixers.
+ZUROLORN_SIZES = {
+    "zurolorn-w2048-h16x128-e32x1024-top8": dict(width=2048, heads=16, dim=128, rot=64, vdim=128, rank=192, q_rank=768, experts=32,
+                                                 ff=1024, top=8, groups=4, keep=2),
+    "zurolorn-w4096-h32x128-e16x3584-top4": dict(width=4096, heads=32, dim=128, rot=64, vdim=128, rank=192, q_rank=1536, experts=16,
+                                                 ff=3584, top=4, groups=4, keep=2),
+}
+
+
+def zurolorn_set(size: dict, layers: int, vocab: int) -> dict[str, dict]:
+    """Name -> config.json of the Zurolorn and of the models it is set beside. ``layers`` is not used: four layer runs."""
+    lat = {"heads": size["heads"], "dim": size["dim"], "rot_dim": size["rot"], "vdim": size["vdim"], "kv_rank": size["rank"],
+           "scale": (size["dim"] + size["rot"]) ** -0.5, "rot": {"base": 10000.0, "dims": size["rot"]}}
+    router = {"experts": size["experts"], "top": size["top"]}
+    mlp = {"kind": "moe", "expert": {"ff": size["ff"]},
+           "router": {**router, "scale": 2.5, "groups": {"count": size["groups"], "keep": size["keep"]}}}
+    one = {"type": "latent_attention", "mixer": lat, "mlp": mlp}
+    two = {"type": "latent_attention_2", "mixer": {**lat, "q_rank": size["q_rank"]}, "mlp": mlp}
+    inner = size["top"] * size["ff"]
+    common = {"vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6}}
+    gokolix = {"architecture": "Gokolix", **common, "embedding": {"scale": 8.0},
+               "layers": [{"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": inner}}] * 4}
+    att = {"heads": size["heads"], "kv_heads": size["heads"] // 4, "dim": size["dim"], "vdim": size["vdim"], "scale": size["dim"] ** -0.5,
+           "rot": {"base": 10000.0, "dims": size["dim"]}}
+    radivik = {"architecture": "Radivik", **common, "postln_alpha": 2.0,
+               "layers": [{"type": "attention", "mixer": att, "mlp": {"kind": "moe", "router": router, "expert": {"ff": size["ff"], "limit": 7.0}}}] * 4}
+    llama = dict(LLAMA_1B, vocab_size=vocab, hidden_size=size["width"], intermediate_size=inner, num_hidden_layers=4,
+                 num_attention_heads=size["heads"], num_key_value_heads=size["heads"] // 4, head_dim=size["dim"], tie_word_embeddings=False)
+    zurolorn = {"architecture": "Zurolorn", **common, "embedding": {"scale": 8.0}, "logit_scale": 0.5, "layers": [two, one, two],
+                "loop": {"start": 1, "stop": 2, "times": 2}}
+    return {"zurolorn": zurolorn, "gokolix": gokolix, "radivik": radivik, "llama": llama}
+
+
 def compare_designs(args) -> int:
-    """Prefill and decode throughput of another design's layers (Radivik, Gokolix, Larupel, Fubelorn) beside Llama layers of
-    equal size, through the same runner and step function. One JSON line; the default benchmark is not run."""
+    """Prefill and decode throughput of another design's layers (Radivik, Gokolix, Larupel, Fubelorn, Zurolorn) beside Llama
+    layers of equal size (Zurolorn: also beside the designs that share its parts), through the same runner and step
+    function. One JSON line; the default benchmark is not run."""
     import numpy as np
     import torch
 
@@ -208,7 +245,10 @@ def compare_designs(args) -> int:
     rng = np.random.default_rng(0)
     vocab, layers = 32000, args.layers or 4
     prompt, batch, context = args.prompt_len, args.batch, args.context
-    if args.compare in FUBELORN_SIZES or args.compare == "fubelorn":
+    if args.compare in ZUROLORN_SIZES or args.compare == "zurolorn":
+        design, pair_of = "zurolorn", None
+        sizes = ZUROLORN_SIZES if args.compare == "zurolorn" else {args.compare: ZUROLORN_SIZES[args.compare]}
+    elif args.compare in FUBELORN_SIZES or args.compare == "fubelorn":
         design, pair_of = "fubelorn", fubelorn_pair
         sizes = FUBELORN_SIZES if args.compare == "fubelorn" else {args.compare: FUBELORN_SIZES[args.compare]}
     elif args.compare in LARUPEL_SIZES or args.compare == "larupel":
@@ -276,15 +316,19 @@ def compare_designs(args) -> int:
 
     with tempfile.TemporaryDirectory(prefix="psamd_compare_") as tmp:
         for name, size in sizes.items():
-            other, llama = pair_of(size, layers, vocab)
+            if pair_of is None:
+                configs = zurolorn_set(size, layers, vocab)
+            else:
+                other, llama = pair_of(size, layers, vocab)
+                configs = {design: other, "llama": llama}
             results[name] = {}
-            for which, cfg in ((design, other), ("llama", llama)):
+            for which, cfg in configs.items():
                 if args.compare_only not in ("both", which):
                     continue
                 folder = write_random_model(Path(tmp) / f"{name}-{which}", cfg, seed=0)
                 results[name][which] = measure(folder)
             both = results[name]
-            if len(both) == 2:
+            if len(both) == len(configs):
                 both[f"{design}_over_llama"] = {k: both[design][k] / both["llama"][k] for k in ("prefill_tok_s", "decode_tok_s")}
     print(json.dumps({"metric": f"{design}_beside_llama_of_equal_size", "unit": "tok/s", "n_gpus": 1, "dtype": args.dtype,
                       "data": "synthetic: seeded uniform-random token ids, seeded random weights",
@@ -331,11 +375,11 @@ def main() -> int:
     ap.add_argument("--model", default=None, help="use this model folder instead of writing random weights")
     ap.add_argument("--shape", choices=sorted(SHAPES), default="llama-3.2-1b", help="layer sizes of the random model")
     ap.add_argument("--compare", choices=sorted(RADIVIK_SIZES) + ["all"] + sorted(GOKOLIX_SIZES) + ["gokolix"] + sorted(LARUPEL_SIZES) + ["larupel"]
-                    + sorted(FUBELORN_SIZES) + ["fubelorn"], default=None,
-                    help="instead of the benchmark: Radivik, Gokolix, Larupel or Fubelorn layers of this size ('all': every Radivik size, "
-                         "'gokolix' / 'larupel' / 'fubelorn': every size of that design) beside Llama layers of equal size (prefill of --prompt-len tokens, "
+                    + sorted(FUBELORN_SIZES) + ["fubelorn"] + sorted(ZUROLORN_SIZES) + ["zurolorn"], default=None,
+                    help="instead of the benchmark: Radivik, Gokolix, Larupel, Fubelorn or Zurolorn layers of this size ('all': every Radivik "
+                         "size, 'gokolix' / 'larupel' / 'fubelorn' / 'zurolorn': every size of that design) beside Llama layers of equal size (prefill of --prompt-len tokens, "
                          "decoding at --batch in --context; --layers, default 4, for Radivik)")
-    ap.add_argument("--compare-only", choices=["both", "radivik", "gokolix", "larupel", "fubelorn", "llama"], default="both")
+    ap.add_argument("--compare-only", choices=["both", "radivik", "gokolix", "larupel", "fubelorn", "zurolorn", "llama"], default="both")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")

@@ -145,6 +145,21 @@ def route(h: np.ndarray, w_router: np.ndarray, r: dict) -> tuple[np.ndarray, np.
     return chosen, np.take_along_axis(s, chosen, axis=1) * r.get("scale", 1.0)
 
 
+def choice_margin(scores: np.ndarray, top: int, groups: dict | None) -> float:
+    """How far the scores of one token would have to move for another choice: the distance between the last
+    kept and the first dropped group, or the last chosen and the first unchosen expert, whichever is less."""
+    margin, allowed = np.inf, np.ones(len(scores), dtype=bool)
+    if groups:
+        per = len(scores) // groups["count"]
+        sums = np.sort(scores.reshape(groups["count"], per), axis=1)[:, ::-1][:, :2].sum(1)
+        order = np.argsort(-sums, kind="stable")
+        if groups["keep"] < groups["count"]:
+            margin = sums[order[groups["keep"] - 1]] - sums[order[groups["keep"]]]
+        allowed = np.isin(np.arange(len(scores)) // per, order[: groups["keep"]])
+    inside = np.sort(scores[allowed])[::-1]
+    return float(min(margin, inside[top - 1] - inside[top] if top < len(inside) else np.inf))
+
+
 def expert(h: np.ndarray, up: np.ndarray, down: np.ndarray, rnd=exact) -> np.ndarray:
     return rnd(np.square(np.maximum(h @ up.T, 0.0))) @ down.T
 
@@ -170,6 +185,7 @@ class PlainZurolorn:
         self.w = load_tensors(folder)
         self.eps = float(self.cfg["norm"]["eps"])
         self.rnd = to_bf16 if bf16 else exact
+        self.margins: list[np.ndarray] = []      # of every layer run with experts of the last call, [T] each
 
     def part(self, prefix: str) -> dict:
         return {k[len(prefix):]: v for k, v in self.w.items() if k.startswith(prefix)}
@@ -183,7 +199,9 @@ class PlainZurolorn:
         x = x + self.w[f"l{i}.ls1"] * self.mixer(i, self.rnd(rms_norm(x, self.w[f"l{i}.norm1"], self.eps)), pos)
         if entry.get("mlp") is not None:
             h = self.rnd(rms_norm(x, self.w[f"l{i}.norm2"], self.eps))
-            x = x + self.w[f"l{i}.ls2"] * mixture(h, self.part(f"l{i}.mlp."), entry["mlp"]["router"], self.rnd)
+            w, r = self.part(f"l{i}.mlp."), entry["mlp"]["router"]
+            x = x + self.w[f"l{i}.ls2"] * mixture(h, w, r, self.rnd)
+            self.margins.append(np.array([choice_margin(s, r["top"], r.get("groups")) for s in sigmoid(h @ w["router"].T)]))
         return x
 
     def runs(self) -> list[tuple[int, int | None]]:
@@ -200,12 +218,18 @@ class PlainZurolorn:
         toks = np.asarray(tokens)
         pos = np.arange(len(toks))
         x, seen = self.w["embed"][toks] * float(self.cfg["embedding"]["scale"]), []
+        self.margins = []
         for i, opens in self.runs():
             if opens is not None:
                 x = x + self.w["loop.step"][opens]
             x = self.layer(i, x, pos)
             seen.append(x)
         return seen if every_layer else x
+
+    def close_calls(self, tokens, below: float, last: int = 0) -> int:
+        """How many (of the ``last``, or all) tokens have an expert choice somewhere that hangs on less than ``below``."""
+        self.hidden(tokens)
+        return int((np.min(self.margins, axis=0)[-last:] < below).sum()) if self.margins else 0
 
     def logits(self, tokens) -> np.ndarray:
         x = self.rnd(rms_norm(self.hidden(tokens), self.w["final.norm"], self.eps))
