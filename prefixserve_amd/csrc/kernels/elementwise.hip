@@ -17,14 +17,14 @@ void set_error(const std::string& msg) { g_error = msg; }
 
 template <typename W>
 __global__ void embed_kernel(const int32_t* __restrict__ ids, const W* __restrict__ table,
-                             float* __restrict__ out, int hidden, int vocab) {
+                             float* __restrict__ out, int hidden, int vocab, float factor) {
   const int64_t t = blockIdx.x;
   // Ids are checked on the host, except those a previous step sampled and left on the device:
   // an id outside the table reads its nearest row instead of memory that is not the table's.
   const int id = min(max(ids[t], 0), vocab - 1);
   const W* row = table + static_cast<int64_t>(id) * hidden;
   float* o = out + t * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_float<W>(row[i]);
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = factor * to_float<W>(row[i]);
 }
 
 // ------------------------------------------------------------------ add + rmsnorm
@@ -629,6 +629,44 @@ __global__ void residual_add_kernel(float* __restrict__ residual, const DT* __re
   }
 }
 
+// The same for widths that are a multiple of 4, four columns a thread: all slices' loads in flight together.
+template <typename DT>
+__global__ __launch_bounds__(256) void residual_add_vec4_kernel(float* __restrict__ residual, const DT* __restrict__ delta, int n_partials,
+                                                                int64_t partial_stride, int64_t n4, const float* __restrict__ scale,
+                                                                const float* __restrict__ row, int hidden) {
+  for (int64_t i = blockIdx.x * 256LL + threadIdx.x; i < n4; i += gridDim.x * 256LL) {
+    const int64_t e = 4 * i;
+    const int col = static_cast<int>(e % hidden);
+    float4 r = *reinterpret_cast<const float4*>(residual + e);
+    float4 sum = scale != nullptr ? float4{0.f, 0.f, 0.f, 0.f} : r;
+    if (sizeof(DT) == 2) {
+      const uint2 q = *reinterpret_cast<const uint2*>(delta + e);
+      sum.x += __uint_as_float(q.x << 16); sum.y += __uint_as_float(q.x & 0xffff0000u);
+      sum.z += __uint_as_float(q.y << 16); sum.w += __uint_as_float(q.y & 0xffff0000u);
+    } else {
+      for (int p = 0; p < n_partials; p += 8) {
+        float4 x[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) x[u] = *reinterpret_cast<const float4*>(delta + min(p + u, n_partials - 1) * partial_stride + e);
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+          if (p + u < n_partials) {
+            sum.x += x[u].x; sum.y += x[u].y; sum.z += x[u].z; sum.w += x[u].w;
+          }
+      }
+    }
+    if (scale != nullptr) {
+      const float4 sc = *reinterpret_cast<const float4*>(scale + col);
+      sum = float4{fmaf(sc.x, sum.x, r.x), fmaf(sc.y, sum.y, r.y), fmaf(sc.z, sum.z, r.z), fmaf(sc.w, sum.w, r.w)};
+    }
+    if (row != nullptr) {
+      const float4 a = *reinterpret_cast<const float4*>(row + col);
+      sum = float4{sum.x + a.x, sum.y + a.y, sum.z + a.z, sum.w + a.w};
+    }
+    *reinterpret_cast<float4*>(residual + e) = sum;
+  }
+}
+
 __global__ void stream_affine_kernel(float* __restrict__ x, int64_t n, int hidden, float factor,
                                      const float* __restrict__ row) {
   for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < n;
@@ -658,14 +696,16 @@ extern "C" {
 const char* psamd_last_error(void) { return g_error.c_str(); }
 
 int psamd_embed(void* stream, const int32_t* ids, const void* table, int table_dtype, float* out, int64_t tokens,
-                int hidden, int vocab) {
+                int hidden, int vocab, float factor) {
   PSAMD_REQUIRE(tokens >= 0 && hidden > 0 && vocab > 0, "bad sizes");
   if (tokens == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (table_dtype == kBF16) {
-    embed_kernel<bf16_t><<<dim3(tokens), dim3(256), 0, s>>>(ids, static_cast<const bf16_t*>(table), out, hidden, vocab);
+    embed_kernel<bf16_t><<<dim3(tokens), dim3(256), 0, s>>>(ids, static_cast<const bf16_t*>(table), out, hidden, vocab,
+                                                            factor);
   } else if (table_dtype == kF32) {
-    embed_kernel<float><<<dim3(tokens), dim3(256), 0, s>>>(ids, static_cast<const float*>(table), out, hidden, vocab);
+    embed_kernel<float><<<dim3(tokens), dim3(256), 0, s>>>(ids, static_cast<const float*>(table), out, hidden, vocab,
+                                                           factor);
   } else {
     return fail("psamd_embed: table dtype must be float32 or bfloat16");
   }
@@ -883,6 +923,19 @@ int psamd_residual_add(void* stream, float* residual, const void* delta, int del
   PSAMD_REQUIRE(n_partials == 1 || delta_dtype == kF32, "partial sums are float32");
   if (rows == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
+  const auto aligned = [](const void* q) { return reinterpret_cast<uintptr_t>(q) % 16 == 0; };
+  if (hidden % 4 == 0 && partial_stride % 4 == 0 && aligned(residual) && aligned(delta) && aligned(scale) && aligned(row) &&
+      (delta_dtype == kBF16 || delta_dtype == kF32)) {
+    const int64_t n4 = rows * hidden / 4;
+    const int grid = static_cast<int>(std::min<int64_t>(ceil_div(n4, 256), 65536));
+    if (delta_dtype == kBF16)
+      residual_add_vec4_kernel<bf16_t><<<dim3(grid), dim3(256), 0, s>>>(residual, static_cast<const bf16_t*>(delta), n_partials,
+                                                                       partial_stride, n4, scale, row, hidden);
+    else
+      residual_add_vec4_kernel<float><<<dim3(grid), dim3(256), 0, s>>>(residual, static_cast<const float*>(delta), n_partials,
+                                                                      partial_stride, n4, scale, row, hidden);
+    return check_launch("psamd_residual_add");
+  }
   const int64_t n = rows * hidden;
   const int blocks = static_cast<int>(std::min<int64_t>(ceil_div(n, 256), 65536));
   if (delta_dtype == kBF16) {

@@ -9,12 +9,13 @@
 // Two forms. LDS-tiled FMA with float accumulation for any element types, the 32-bit path's
 // product: k is summed in ascending order whatever the number of tokens, so a token's 32-bit
 // result does not depend on what else is in the step. And, for bfloat16 operands whose rows start
-// on 16-byte boundaries, v_mfma_f32_16x16x32_bf16 with both operands straight from memory (they
-// are small: a head's matrix stays in L2 for all its tokens): a wave owns 16 tokens and NT tiles
-// of 16 output columns, so the tokens' fragment serves NT matrix instructions.
+// on 16-byte boundaries, the matrix cores (heads_tile.h): a wave owns 16 tokens and NT tiles of 16 output
+// columns, so the tokens' fragment serves NT matrix instructions; with up to 16 tokens in all, the four
+// waves share them and own 16 columns each.
 
 #include "api.h"
 #include "common.h"
+#include "heads_tile.h"
 
 namespace psamd {
 
@@ -74,56 +75,45 @@ __global__ __launch_bounds__(256) void heads_linear_kernel(const TX* __restrict_
   }
 }
 
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
-typedef __attribute__((ext_vector_type(4))) float f32x4;
-
-// Operand layout of the instruction: lane l supplies row l % 16, k = 8 * (l / 16) + [0, 8) of both
-// operands and receives C[4 * (l / 16) + v][l % 16]; C's rows are rows of w, its columns tokens.
-template <int NT>
+// vec: out's heads start on 8-byte boundaries, so four results may be one store.
+template <int NT, int U, bool FEW>
 __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const bf16_t* __restrict__ x, int64_t x_row, int x_head,
                                                                 const bf16_t* __restrict__ w, bf16_t* __restrict__ out,
                                                                 int64_t o_row, int o_head, int64_t M, int N, int K,
-                                                                const bf16_t* __restrict__ gate, int64_t g_row, int g_head) {
+                                                                const bf16_t* __restrict__ gate, int64_t g_row, int g_head,
+                                                                int vec) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
   const int h = blockIdx.z;
-  const int64_t m0 = (static_cast<int64_t>(blockIdx.y) * 4 + wave) * 16;
-  if (m0 >= M) return;
-  const int n0 = blockIdx.x * NT * 16;
-  const bf16_t* xr = x + static_cast<int64_t>(h) * x_head + min(m0 + r, M - 1) * x_row + 8 * g;
+  const HeadPlace<NT, FEW> place(wave);
+  const int n0 = place.n0;
+  if (place.m0 >= M || n0 >= N) return;
   const bf16_t* wr[NT];
 #pragma unroll
-  for (int nt = 0; nt < NT; ++nt)
-    wr[nt] = w + (static_cast<int64_t>(h) * N + min(n0 + nt * 16 + r, N - 1)) * K + 8 * g;
-  f32x4 acc[NT];
-#pragma unroll
-  for (int nt = 0; nt < NT; ++nt) acc[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  bf16x8 zero;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) zero[i] = static_cast<__bf16>(0.f);
-  for (int k0 = 0; k0 < K; k0 += 32) {
-    const bool in = k0 + 8 * g < K;                   // K is a multiple of 8: a piece is inside or outside
-    const bf16x8 b = in ? *reinterpret_cast<const bf16x8*>(xr + k0) : zero;
-#pragma unroll
-    for (int nt = 0; nt < NT; ++nt) {
-      const bf16x8 a = in ? *reinterpret_cast<const bf16x8*>(wr[nt] + k0) : zero;
-      acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[nt], 0, 0, 0);
-    }
-  }
-  const int64_t m = m0 + r;
+  for (int nt = 0; nt < NT; ++nt) wr[nt] = w + (static_cast<int64_t>(h) * N + min(n0 + nt * 16 + r, N - 1)) * K;
+  head_f32x4 acc[NT];
+  head_tile<NT, U>(x + static_cast<int64_t>(h) * x_head + min(place.m0 + r, M - 1) * x_row, wr, K, g, acc);
+  const int64_t m = place.m0 + r;
   if (m >= M) return;
   bf16_t* o = out + static_cast<int64_t>(h) * o_head + m * o_row;
   const bf16_t* gt = gate != nullptr ? gate + static_cast<int64_t>(h) * g_head + m * g_row : nullptr;
 #pragma unroll
-  for (int nt = 0; nt < NT; ++nt)
+  for (int nt = 0; nt < NT; ++nt) {
+    const int n = n0 + nt * 16 + 4 * g;
+    if (gt != nullptr) {
 #pragma unroll
-    for (int v = 0; v < 4; ++v) {
-      const int n = n0 + nt * 16 + 4 * g + v;
-      if (n >= N) continue;
-      float y = acc[nt][v];
-      if (gt != nullptr) y *= 1.f / (1.f + __expf(-bf16_to_float(gt[n])));
-      o[n] = float_to_bf16(y);
+      for (int v = 0; v < 4; ++v)
+        if (n + v < N) acc[nt][v] *= 1.f / (1.f + __expf(-bf16_to_float(gt[n + v])));
     }
+    if (vec && n + 3 < N) {
+      *reinterpret_cast<ushort4*>(o + n) = ushort4{float_to_bf16(acc[nt][0]), float_to_bf16(acc[nt][1]),
+                                                   float_to_bf16(acc[nt][2]), float_to_bf16(acc[nt][3])};
+      continue;
+    }
+#pragma unroll
+    for (int v = 0; v < 4; ++v)
+      if (n + v < N) o[n + v] = float_to_bf16(acc[nt][v]);
+  }
 }
 
 template <typename T>
@@ -153,11 +143,12 @@ extern "C" int psamd_heads_linear(void* stream, const void* x, int x_dtype, int6
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (x_dtype == kBF16 && K % 8 == 0 && x_row % 8 == 0 && x_head % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(w) % 16 == 0 && ceil_div(M, 64) <= 65535) {
-    constexpr int NT = 4;
-    const dim3 grid(static_cast<unsigned>(ceil_div(N, 16 * NT)), static_cast<unsigned>(ceil_div(M, 64)), static_cast<unsigned>(H));
-    heads_linear_mfma_kernel<NT><<<grid, dim3(256), 0, s>>>(static_cast<const bf16_t*>(x), x_row, x_head,
-                                                           static_cast<const bf16_t*>(w), static_cast<bf16_t*>(out), out_row,
-                                                           out_head, M, N, K, static_cast<const bf16_t*>(gate), gate_row, gate_head);
+    const int vec = out_row % 4 == 0 && out_head % 4 == 0 && reinterpret_cast<uintptr_t>(out) % 8 == 0;
+    const dim3 grid(static_cast<unsigned>(ceil_div(N, 64)), static_cast<unsigned>(ceil_div(M, 64)), static_cast<unsigned>(H));
+    auto kernel = M <= 16 ? heads_linear_mfma_kernel<1, 8, true> : heads_linear_mfma_kernel<4, 4, false>;
+    kernel<<<grid, dim3(256), 0, s>>>(static_cast<const bf16_t*>(x), x_row, x_head, static_cast<const bf16_t*>(w),
+                                      static_cast<bf16_t*>(out), out_row, out_head, M, N, K, static_cast<const bf16_t*>(gate), gate_row,
+                                      gate_head, vec);
     return check_launch("psamd_heads_linear");
   }
   if (x_dtype == kBF16) return launch_heads<bf16_t>(s, x, x_row, x_head, w, out, out_row, out_head, M, H, N, K, gate, gate_row, gate_head);

@@ -15,6 +15,7 @@
 
 #include "api.h"
 #include "common.h"
+#include "heads_tile.h"
 
 namespace psamd {
 
@@ -116,13 +117,9 @@ __global__ __launch_bounds__(256) void latent_query_tail_kernel(const A* __restr
   }
 }
 
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
-typedef __attribute__((ext_vector_type(4))) float f32x4;
-
 // Folding and tails in one kernel on the matrix cores: the grid's last column of workgroups lays the
-// tails of its 64 tokens of one head, the others each fold 64 tokens into NT * 16 of the compressed
-// dimensions (operands straight from memory, as in heads_linear's kernel of this form).
-template <int NT>
+// tails of its tokens of one head, the others fold (heads_tile.h).
+template <int NT, int U, bool FEW>
 __global__ __launch_bounds__(256) void latent_query_mfma_kernel(const bf16_t* __restrict__ q_rows, int64_t q_row,
                                                                 const bf16_t* __restrict__ w, bf16_t* __restrict__ q_lat, int64_t M,
                                                                 int hq, int dim, int rot, int rank, int slots, int halves,
@@ -147,36 +144,21 @@ __global__ __launch_bounds__(256) void latent_query_mfma_kernel(const bf16_t* __
   }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
-  const int64_t m0 = (static_cast<int64_t>(blockIdx.y) * 4 + wave) * 16;
-  if (m0 >= M) return;
-  const int n0 = blockIdx.x * NT * 16;
-  const bf16_t* xr = q + min(m0 + r, M - 1) * q_row + 8 * g;
+  const HeadPlace<NT, FEW> place(wave);
+  const int n0 = place.n0;
+  if (place.m0 >= M || n0 >= rank) return;
   const bf16_t* wr[NT];
 #pragma unroll
-  for (int nt = 0; nt < NT; ++nt)
-    wr[nt] = w + (static_cast<int64_t>(h) * rank + min(n0 + nt * 16 + r, rank - 1)) * dim + 8 * g;
-  f32x4 acc[NT];
-#pragma unroll
-  for (int nt = 0; nt < NT; ++nt) acc[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  bf16x8 zero;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) zero[i] = static_cast<__bf16>(0.f);
-  for (int k0 = 0; k0 < dim; k0 += 32) {
-    const bool in = k0 + 8 * g < dim;                 // dim is a multiple of 8: a piece is inside or outside
-    const bf16x8 b = in ? *reinterpret_cast<const bf16x8*>(xr + k0) : zero;
-#pragma unroll
-    for (int nt = 0; nt < NT; ++nt) {
-      const bf16x8 a = in ? *reinterpret_cast<const bf16x8*>(wr[nt] + k0) : zero;
-      acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[nt], 0, 0, 0);
-    }
-  }
-  const int64_t m = m0 + r;
+  for (int nt = 0; nt < NT; ++nt) wr[nt] = w + (static_cast<int64_t>(h) * rank + min(n0 + nt * 16 + r, rank - 1)) * dim;
+  head_f32x4 acc[NT];
+  head_tile<NT, U>(q + min(place.m0 + r, M - 1) * q_row, wr, dim, g, acc);
+  const int64_t m = place.m0 + r;
   if (m >= M) return;
   bf16_t* o = out + m * o_row;
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {
     const int n = n0 + nt * 16 + 4 * g;
-    if (n + 3 < rank) {                               // slots is a multiple of 16: four results are one 8-byte store
+    if (n + 3 < rank) {                               // slots is a multiple of 4: four results are one 8-byte store
       *reinterpret_cast<ushort4*>(o + n) = ushort4{float_to_bf16(acc[nt][0]), float_to_bf16(acc[nt][1]),
                                                    float_to_bf16(acc[nt][2]), float_to_bf16(acc[nt][3])};
     } else {
@@ -246,13 +228,13 @@ int psamd_latent_query(void* stream, const void* q, int64_t q_row, const void* w
   PSAMD_REQUIRE(hq <= 65535 && ceil_div(tokens, 64) <= 65535, "too large for one launch");
   if (tokens == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (act_dtype == kBF16 && dim % 8 == 0 && rot % 8 == 0 && q_row % 8 == 0 && slots % 4 == 0 &&
+  if (act_dtype == kBF16 && dim > 0 && dim % 8 == 0 && rot % 8 == 0 && q_row % 8 == 0 && slots % 4 == 0 &&
       reinterpret_cast<uintptr_t>(q) % 16 == 0 && reinterpret_cast<uintptr_t>(w_fold) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(q_lat) % 8 == 0) {
-    constexpr int NT = 4;
-    const dim3 grid(static_cast<unsigned>(ceil_div(rank, 16 * NT)) + 1, static_cast<unsigned>(ceil_div(tokens, 64)),
+    const dim3 grid(static_cast<unsigned>(ceil_div(rank, 64)) + 1, static_cast<unsigned>(ceil_div(tokens, 64)),
                     static_cast<unsigned>(hq));
-    latent_query_mfma_kernel<NT><<<grid, dim3(256), 0, s>>>(
+    auto kernel = tokens <= 16 ? latent_query_mfma_kernel<1, 4, true> : latent_query_mfma_kernel<4, 4, false>;
+    kernel<<<grid, dim3(256), 0, s>>>(
         static_cast<const bf16_t*>(q), q_row, static_cast<const bf16_t*>(w_fold), static_cast<bf16_t*>(q_lat), tokens, hq, dim, rot,
         rank, slots, halves, positions, reinterpret_cast<const float2*>(table));
     return check_launch("psamd_latent_query");

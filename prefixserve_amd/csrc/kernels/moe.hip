@@ -152,12 +152,64 @@ __device__ __forceinline__ void keep_best_groups(float* score, int experts, int 
   __threadfence_block();
 }
 
+// The same choice for up to 64 experts without LDS: lane e holds expert e's score (lanes past the last hold nothing of
+// use) and counts who comes in front of it.
+__device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top, RouterRule rule, int32_t* __restrict__ chosen,
+                                                  float* __restrict__ weight, int lane) {
+  const float kTaken = -__builtin_inff();
+  auto of = [](float v, int from) { return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), from)); };
+  if (lane >= experts) s = kTaken;
+  if (rule.groups > 0) {
+    const int size = experts / rule.groups, mine = lane / size;
+    float a = kTaken, b = kTaken;                         // the two largest of the lane's own group
+    for (int e = 0; e < experts; ++e) {
+      const float v = of(s, e);
+      if (e / size == mine) {
+        b = fmaxf(b, fminf(a, v));
+        a = fmaxf(a, v);
+      }
+    }
+    const float sum = a + (size > 1 ? b : 0.f);
+    int ahead = 0;                                        // groups in front of the lane's own
+    for (int grp = 0; grp < rule.groups; ++grp) {
+      const float v = of(sum, grp * size);
+      ahead += (v > sum || (v == sum && grp < mine)) ? 1 : 0;
+    }
+    if (ahead >= rule.keep) s = kTaken;
+  }
+  int rank = 0;
+  for (int e = 0; e < experts; ++e) {
+    const float v = of(s, e);
+    rank += (v > s || (v == s && e < lane)) ? 1 : 0;
+  }
+  const bool taken = lane < experts && rank < top && s > kTaken;
+  float w = s;
+  if (rule.mode == 1) {
+    const float m = wave_max(taken ? s : kTaken);
+    // Summed in the order of the choice, largest first.
+    float sum = 0.f;
+    for (int j = 0; j < top; ++j) {
+      const unsigned long long at = __ballot(taken && rank == j);
+      if (at != 0) sum += expf(of(s, __ffsll(static_cast<unsigned long long>(at)) - 1) - m);
+    }
+    w = expf(s - m) / sum;
+  }
+  if (taken) {
+    chosen[rank] = lane;
+    weight[rank] = rule.factor * w;
+  }
+}
+
 // The router's choice for one token by one wave: score[] (LDS, `experts` entries: sigmoid(z) in mode
 // 0, z in mode 1) -> chosen / weight [top], largest first, the lower index among equals; taken
 // entries are overwritten. Mode 1 then turns the chosen z into their softmax.
 __device__ __forceinline__ void pick_top(float* score, int experts, int top, RouterRule rule, int32_t* __restrict__ chosen,
                                          float* __restrict__ weight, int lane) {
   const float kTaken = -__builtin_inff();
+  if (experts <= kWave) {
+    pick_top_in_lanes(lane < experts ? score[lane] : 0.f, experts, top, rule, chosen, weight, lane);
+    return;
+  }
   if (rule.groups > 0) keep_best_groups(score, experts, rule.groups, rule.keep, lane);
   for (int j = 0; j < top; ++j) {
     float best = kTaken;
@@ -315,15 +367,29 @@ __device__ __forceinline__ void group_pairs(const int32_t* __restrict__ chosen, 
   __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += blockDim.x) atomicAdd(&count[min(max(chosen[p], 0), experts - 1)], 1);
   __syncthreads();
-  if (threadIdx.x == 0) {
-    int at = 0, nt = 0;
-    for (int e = 0; e < experts; ++e) {
-      start[e] = at;
-      tstart[e] = nt;
-      at += count[e];
-      nt += (count[e] + tile_rows - 1) / tile_rows;
+  if (threadIdx.x < kWave) {                     // where every expert's pairs and tiles begin: sums over the wave's lanes
+    const int lane = threadIdx.x;
+    int at = 0, nt = 0;                          // of the experts in front of this run of 64
+    for (int e0 = 0; e0 < experts; e0 += kWave) {
+      const int e = e0 + lane;
+      const int pairs_e = e < experts ? count[e] : 0, tiles_e = (pairs_e + tile_rows - 1) / tile_rows;
+      int p_sum = pairs_e, t_sum = tiles_e;
+#pragma unroll
+      for (int o = 1; o < kWave; o <<= 1) {
+        const int p_up = __shfl_up(p_sum, o, kWave), t_up = __shfl_up(t_sum, o, kWave);
+        if (lane >= o) {
+          p_sum += p_up;
+          t_sum += t_up;
+        }
+      }
+      if (e < experts) {
+        start[e] = at + p_sum - pairs_e;
+        tstart[e] = nt + t_sum - tiles_e;
+      }
+      at += __shfl(p_sum, kWave - 1, kWave);
+      nt += __shfl(t_sum, kWave - 1, kWave);
     }
-    *n_tiles = min(nt, max_tiles);
+    if (lane == 0) *n_tiles = min(nt, max_tiles);
   }
   __syncthreads();
   for (int e = threadIdx.x; e < experts; e += blockDim.x) {
@@ -373,8 +439,9 @@ __global__ __launch_bounds__(1024) void moe_topk_group_kernel(const float* __res
               group_smem + experts, group_smem + 2 * experts, group_smem + 3 * experts, group_smem + 4 * experts);
 }
 
-constexpr int kGroupBK = 64;                   // k per staging round
-constexpr int kGroupLD = kGroupBK + 8;         // LDS row stride of the staged pairs, in elements
+// k per staging round: with one tile of pairs a round of 64 leaves a wave two pieces of its matrix in flight, too few to
+// hide a trip to memory.
+constexpr int group_bk(int mt) { return mt == 1 ? 128 : 64; }
 
 // One workgroup (4 waves) per (64 * RT output columns, tile of MT * 16 pairs of one expert). The
 // pairs' input rows pass through LDS 64 k at a time (gathered through `sorted`). GATED: the
@@ -398,6 +465,8 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     int K, int N, int top, float gate_alpha, float limit, float up_shift, int into_stream,
     const float* __restrict__ col_scale) {
   constexpr bool GATED = FORM == kFormGated;
+  constexpr int kGroupBK = group_bk(MT);
+  constexpr int kGroupLD = kGroupBK + 8;                     // LDS row stride of the staged pairs, in elements
   constexpr int ROWS = MT * 16;
   constexpr int PIECES = ROWS * (kGroupBK / 8);              // 16-byte pieces of a round's pairs
   constexpr int PPT = (PIECES + 255) / 256;                  // pieces per thread

@@ -49,6 +49,8 @@ class DecoderModel:
         self.final_norm = make("norm", spec.final_norm.kind, hidden_size=spec.hidden_size, **spec.final_norm.params)
         sizes = dict(hidden_size=spec.hidden_size, vocab_size=spec.vocab_size)
         self.embedding_transforms = [make("transform", ps.kind, **sizes, **ps.params) for ps in spec.embedding_transforms]
+        # A constant in front of everything else is the gather's own factor.
+        self.embedding_factor = getattr(self.embedding_transforms[0], "embedding_factor", None) if self.embedding_transforms else None
         self.logit_transforms = [make("transform", ps.kind, **sizes, **ps.params) for ps in spec.logit_transforms]
         self.stream_transforms = {name: make("transform", ps.kind, **sizes, **ps.params)
                                   for name, ps in spec.stream_transforms.items()}
@@ -181,8 +183,11 @@ class DecoderModel:
                 residual = streams[0]
             else:
                 streams = residual = ws.get("residual", (t, s.hidden_size), torch.float32)
-            ops.embed(ctx.token_ids, self.embedding, residual)
-            for tr in self.embedding_transforms:
+            if self.embedding_factor is not None:
+                ops.embed(ctx.token_ids, self.embedding, residual, factor=self.embedding_factor)
+            else:
+                ops.embed(ctx.token_ids, self.embedding, residual)
+            for tr in self.embedding_transforms[0 if self.embedding_factor is None else 1:]:
                 tr.apply(residual, ctx, None)
             if s.streams > 1:
                 streams[1:].copy_(residual.unsqueeze(0).expand(s.streams - 1, t, s.hidden_size))

@@ -14,10 +14,11 @@ if TYPE_CHECKING:
 
 
 class ScaleStream(Transform):
-    """t <- factor * t, in 32-bit: the token table's rows times a constant."""
+    """t <- factor * t, in 32-bit: the token table's rows, or the logits, times a constant. As the first
+    transform behind the token table it is applied by the gather (``embedding_factor``)."""
 
     def __init__(self, hidden_size: int, vocab_size: int, factor: float) -> None:
-        self.factor = float(factor)
+        self.factor = self.embedding_factor = float(factor)
 
     def apply(self, t: torch.Tensor, ctx: "StepContext", rows: torch.Tensor | None) -> None:
         if self.factor != 1.0:

@@ -32,8 +32,8 @@ class EmulatedOps:
     def prepare_matrix(self, w: torch.Tensor, rt) -> torch.Tensor:
         return w.to(device=rt.device, dtype=rt.dtype).contiguous()
 
-    def embed(self, ids, table, out) -> None:
-        out.copy_(table[ids.long()].float())
+    def embed(self, ids, table, out, factor=1.0) -> None:
+        out.copy_(table[ids.long()].float() * factor)
 
     @staticmethod
     def _whole(delta):
