@@ -1,5 +1,5 @@
 // Causal grouped-query attention over the paged cache, the straightforward way: one wave
-// per (new token, query head), float arithmetic throughout, any head size up to 512, any number
+// per (new token, query head), float arithmetic throughout, any head size up to 1,024, any number
 // of heads and groups, optional sliding window, an optional
 // learned sink per head (a term exp(sink) in the softmax's denominator that has no key and no
 // value) and an optional bias on the scaled score that depends on the head and on how far back
@@ -15,7 +15,7 @@
 
 namespace psamd {
 
-constexpr int kMaxHead = 512;          // head sizes up to here: kMaxHead / 64 output dimensions per lane
+constexpr int kMaxHead = 1024;         // head sizes up to here: kMaxHead / 64 output dimensions per lane
 
 template <typename A>
 __global__ __launch_bounds__(64) void attention_generic_kernel(
@@ -196,7 +196,7 @@ extern "C" int psamd_attention_generic(void* stream, const void* qkv, int q_stri
                                        const float* dist_bias, int n_dist) {
   PSAMD_REQUIRE(dist_bias == nullptr || n_dist >= 1, "a distance bias needs at least one entry per head");
   PSAMD_REQUIRE(tokens >= 0 && hq > 0 && hkv > 0 && hq % hkv == 0, "bad head counts");
-  PSAMD_REQUIRE(head_dim > 0 && head_dim <= kMaxHead, "head_dim must be in [1, 512]");
+  PSAMD_REQUIRE(head_dim > 0 && head_dim <= kMaxHead, "head_dim must be in [1, 1024]");
   PSAMD_REQUIRE(hq <= 65535, "too many heads for one launch");
   if (tokens == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -222,7 +222,7 @@ extern "C" int psamd_attention_masked(void* stream, const void* qkv, int q_strid
                                       const int32_t* pool_table_off, const int32_t* pool_block_ids, int block,
                                       const float* gate) {
   PSAMD_REQUIRE(tokens >= 0 && hq > 0 && hkv > 0 && hq % hkv == 0, "bad head counts");
-  PSAMD_REQUIRE(head_dim > 0 && head_dim <= kMaxHead, "head_dim must be in [1, 512]");
+  PSAMD_REQUIRE(head_dim > 0 && head_dim <= kMaxHead, "head_dim must be in [1, 1024]");
   PSAMD_REQUIRE(hq <= 65535, "too many heads for one launch");
   PSAMD_REQUIRE(window >= 1 && keep_first >= 0, "kept first positions and pooled blocks belong to a window");
   PSAMD_REQUIRE(pool == nullptr || (block >= 1 && pool_table_off != nullptr && pool_block_ids != nullptr),

@@ -162,13 +162,14 @@ __device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top,
   if (rule.groups > 0) {
     const int size = experts / rule.groups, mine = lane / size;
     float a = kTaken, b = kTaken;                         // the two largest of the lane's own group
-    for (int e = 0; e < experts; ++e) {
-      const float v = of(s, e);
-      if (e / size == mine) {
-        b = fmaxf(b, fminf(a, v));
-        a = fmaxf(a, v);
+    for (int grp = 0; grp < rule.groups; ++grp)
+      for (int i = 0; i < size; ++i) {
+        const float v = of(s, grp * size + i);
+        if (grp == mine) {
+          b = fmaxf(b, fminf(a, v));
+          a = fmaxf(a, v);
+        }
       }
-    }
     const float sum = a + (size > 1 ? b : 0.f);
     int ahead = 0;                                        // groups in front of the lane's own
     for (int grp = 0; grp < rule.groups; ++grp) {

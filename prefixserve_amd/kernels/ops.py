@@ -138,6 +138,7 @@ class HipOps:
     FUSED_SWIGLU_MAX_ROWS = 32      # above it (to SKINNY_MAX_ROWS) gate/up goes to the library, where there is one
     LIBRARY_ADD_MIN_ROWS = 1024     # from here on a product that feeds the residual stream adds into it in the library
     MOE_ROUTE_FUSED_MAX_TOKENS = 0   # up to here one kernel computes router logits and choice; above, product + choice
+    MOE_CHOICE_SORTS_MAX_TOKENS = 16 # up to here the workgroup that chooses a step's experts also sorts the pairs
     MOE_PAIRWISE_MAX_TOKENS = 2     # up to here a bfloat16 step's experts run pair by pair; above, grouped by expert
     MFMA_ATTENTION_EXTRAS = True    # whether the matrix-core attention takes a sink and a bias by distance
     name = "hip"
@@ -768,7 +769,7 @@ class HipOps:
             logits = self.ws.get("moe.logits", (t, e), torch.float32)
             self.linear(x, w_router_act, logits)
             self._grouped_for = None
-            if self._groups_pairs(x.dtype, t, k) and t <= 64 and e <= 1024:
+            if self._groups_pairs(x.dtype, t, k) and t <= self.MOE_CHOICE_SORTS_MAX_TOKENS and e <= 1024:
                 # A small step: the workgroup that chooses also sorts the pairs for the experts' kernels.
                 ints = self._group_ints(t, top, e)
                 self._ok(self.lib.psamd_moe_topk_group(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(),

@@ -33,10 +33,10 @@ class LayerCache:
 def slot_size(head_dim: int, value_dim: int, largest: int = 256) -> int:
     """The head size the pages and kernels run with: the larger of the two sizes, rounded up to
     one the matrix-core attention takes (multiples of 16 up to 128, then 160, 192, 256). A mixer
-    whose other kernels take more may allow up to 512 (``largest``): sizes above 256 are multiples
+    whose other kernels take more may allow up to 1,024 (``largest``): sizes above 256 are multiples
     of 64 and run the attention kernel of the 32-bit path in either dtype."""
     need = max(int(head_dim), int(value_dim))
-    for size in (*range(16, 129, 16), 160, 192, 256, 320, 384, 448, 512):
+    for size in (*range(16, 129, 16), 160, 192, 256, *range(320, 1025, 64)):
         if need <= size <= largest:
             return size
     raise ValueError(f"head sizes up to {largest} are implemented, got {need}")

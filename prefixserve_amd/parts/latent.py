@@ -59,7 +59,7 @@ class LatentAttention(Mixer):
             if not isinstance(self.pos, RotaryTable) or self.pos.head_dim != self.rot_dim \
                     or (self.pos.rotary_dim or self.rot_dim) != self.rot_dim:
                 raise ValueError(f"the rotated part needs a rotation table of {self.rot_dim} dimensions")
-        self.slots = slot_size(self.rank + self.rot_dim, self.rank, largest=512)
+        self.slots = slot_size(self.rank + self.rot_dim, self.rank, largest=1024)
         self.q_width = self.num_heads * (self.head_dim + self.rot_dim)
         # Columns of the input product: queries (or their latent), the compressed vector with the shared part, the gate.
         self.low_col = self.q_width if self.q_rank is None else self.q_rank

@@ -358,10 +358,11 @@ def test_long_contexts_and_far_keys(dtype, tmp_path):
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_sizes_at_the_kernels_limits(dtype, tmp_path):
-    """A cache entry of 256 and one wider than the matrix-core attention takes, a queries' latent wider than
-    the model, 256 experts in 128 groups, a head of 256 value dimensions."""
+    """A cache entry of 256 and ones wider than the matrix-core attention takes (332 and 576 numbers), a queries'
+    latent wider than the model, 256 experts in 128 groups, a head of 256 value dimensions."""
     cfg = model(90, 128, 1e-5, 2.0, 1.0, [layer(latent(2, 64, 64, 256, 192, 0.1, 1e4), moe(256, 6, 16, 2.0, (128, 5))),
-                                          layer(latent(3, 32, 32, 16, 300, 0.1, 1e4, q_rank=200), moe(2, 2, 200, 1.0, (1, 1)))])
+                                          layer(latent(3, 32, 32, 16, 300, 0.1, 1e4, q_rank=200), moe(2, 2, 200, 1.0, (1, 1))),
+                                          layer(latent(2, 16, 64, 16, 512, 0.1, 1e4), None)])
     folder = write_zurolorn(tmp_path, cfg, seed=9)
     toks = np.random.default_rng(5).integers(0, 90, 60).tolist()
     truth = plain.PlainZurolorn(folder).logits(toks)
