@@ -1,3 +1,4 @@
+from .durelix import DurelixConfig
 from .fubelorn import FubelornConfig
 from .gokolix import GokolixConfig
 from .larupel import LarupelConfig
@@ -8,7 +9,7 @@ from .registry import (Architecture, UnknownArchitectureError, architecture_of, 
 from .zurolorn import ZurolornConfig
 
 __all__ = [
-    "Architecture", "FubelornConfig", "GokolixConfig", "LarupelConfig", "Llama3RopeScaling", "LlamaConfig", "RadivikConfig", "UnknownArchitectureError", "UnsupportedModelError",
+    "Architecture", "DurelixConfig", "FubelornConfig", "GokolixConfig", "LarupelConfig", "Llama3RopeScaling", "LlamaConfig", "RadivikConfig", "UnknownArchitectureError", "UnsupportedModelError",
     "ZurolornConfig",
     "architecture_of", "read_model_dir", "register_architecture", "registered_architectures",
 ]

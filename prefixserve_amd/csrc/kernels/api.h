@@ -124,21 +124,26 @@ int psamd_gated_scan(void* stream, const float* gates, const float* gate_b, cons
 // first), weight[t, :] = those scores. bias (float [experts] or NULL) is added to z first. mode 1: the
 // choice is by z itself and the weights are the softmax over the chosen z alone. groups > 0 (mode 0): the
 // experts form that many equal runs of neighbours, a run's score is the sum of its two largest scores,
-// and only experts of the `keep` best runs can be chosen. The weights are multiplied by factor.
+// and only experts of the `keep` best runs can be chosen. The weights are multiplied by factor. mode 2: the scores are
+// the softmax over all z, the choice goes by score + correction (float [experts] or NULL), the weights are the scores;
+// groups go with it too. group_max: a run's score is its largest score alone.
 int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_router, int32_t* chosen, float* weight,
-                    int64_t tokens, int K, int experts, int top, const float* bias, int mode, int groups, int keep, float factor);
+                    int64_t tokens, int K, int experts, int top, const float* bias, int mode, int groups, int keep, float factor, int group_max,
+                    const float* correction);
 // The same choice from logits that a product has written (float [tokens, experts]).
 int psamd_moe_topk(void* stream, const float* logits, int32_t* chosen, float* weight, int64_t tokens, int experts,
-                   int top, const float* bias, int mode, int groups, int keep, float factor);
+                   int top, const float* bias, int mode, int groups, int keep, float factor, int group_max,
+                    const float* correction);
 // Experts, one (token, choice) pair at a time: h = weight[t, j] * x[t]; g = min(gate h, limit), u =
 // clamp(up h, -limit, limit); act[t * top + j] = g * sigmoid(gate_alpha * g) * (u + up_shift);
 // out[j][t] = down act (float). w_in is [E, 2F, K] (gate rows, then up rows), w_down [E, K, F].
 // weight_on_output: h = x[t] and out[j][t] = weight[t, j] * down act instead. kind 1: no gate, act = max(up h, 0)^2,
 // w_in is [E, F, K]. into_stream: out is [tokens, K] and every pair adds its output into it, times col_scale
-// (float [K] or NULL), with float atomics.
+// (float [K] or NULL), with float atomics. Choices from `experts` on (`identity` of them) are identity experts: their
+// output is weight[t, j] * x[t].
 int psamd_moe_experts_rows(void* stream, const void* x, const int32_t* chosen, const float* weight,
                            const void* w_in, const void* w_down, void* act, float* out, int dtype,
-                           int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
+                           int64_t tokens, int K, int F, int experts, int identity, int top, float gate_alpha, float limit,
                            float up_shift, int weight_on_output, int kind, int into_stream, const float* col_scale);
 
 // The same for bfloat16 with the pairs sorted by expert and every expert's pairs run through its
@@ -148,13 +153,15 @@ int psamd_moe_grouped_tile_rows(int64_t pairs, int experts);
 int psamd_moe_grouped_max_tiles(int64_t pairs, int experts);
 int psamd_moe_experts_grouped(void* stream, const void* x, const int32_t* chosen, const float* weight,
                               const void* w_in, const void* w_down, void* act, float* out, int32_t* ints,
-                              int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
+                              int64_t tokens, int K, int F, int experts, int identity, int top, float gate_alpha, float limit,
                               float up_shift, int grouped_already, int weight_on_output, int kind, int into_stream,
                               const float* col_scale);
-// psamd_moe_topk and the sorting of the pairs into `ints` in one workgroup, for up to 64 tokens;
+// psamd_moe_topk and the sorting of the pairs into `ints` in one workgroup, for up to 64 tokens (buckets: the experts with
+// matrices, plus one if there are identity experts; psamd_moe_grouped_max_tiles then takes buckets for experts);
 // psamd_moe_experts_grouped is then called with grouped_already = 1 and the same `ints`.
 int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, float* weight, int32_t* ints, int64_t tokens,
-                         int experts, int top, const float* bias, int mode, int groups, int keep, float factor);
+                         int experts, int buckets, int top, const float* bias, int mode, int groups, int keep, float factor, int group_max,
+                    const float* correction);
 // out[t, :] *= sigmoid(x[t] . w) for float out [tokens, out_hidden], x [tokens, hidden] in act_dtype, w float [hidden].
 int psamd_row_gate(void* stream, float* out, const void* x, int act_dtype, const float* w, int64_t tokens, int out_hidden,
                    int hidden);
@@ -313,7 +320,8 @@ int psamd_qkv_rope_append_normed(void* stream, const float* resid, const void* n
 int psamd_attention_generic(void* stream, const void* qkv, int q_stride, void* out, const void* kv, int act_dtype,
                             int64_t tokens, const int32_t* positions, const int32_t* tok_item,
                             const int32_t* table_off, const int32_t* block_ids, int hq, int hkv, int head_dim,
-                            float scale, int window, const float* sink, const float* dist_bias, int n_dist);
+                            float scale, int window, const float* sink, const float* dist_bias, int n_dist,
+                            const void* gate, int64_t gate_row);
 
 int psamd_attention_mfma_supports(int hq, int hkv, int head_dim);
 
@@ -349,18 +357,57 @@ int psamd_attention_decode(void* stream, const void* qkv, int q_stride, void* ou
                            int exact_weights);
 
 // psamd_attention_prefill and psamd_attention_decode with a sink and a bias by distance (see
-// psamd_attention_generic for both; either may be NULL).
+// psamd_attention_generic for both; either may be NULL) and the gate on the output.
 int psamd_attention_prefill_extras(void* stream, const void* qkv, int q_stride, void* out, const void* kv,
                                    const int32_t* pf_tiles, int n_tiles, const int32_t* pf_blocks, int n_blocks,
                                    int max_kv_len, const int32_t* item_start, const int32_t* item_pos0,
                                    const int32_t* table_off, const int32_t* block_ids, int hq, int hkv, int head_dim,
                                    float scale, int window, float* part_o, float* part_ml, int nsplit, int exact_weights,
-                                   const float* sink, const float* dist_bias, int n_dist);
+                                   const float* sink, const float* dist_bias, int n_dist,
+                            const void* gate, int64_t gate_row);
 int psamd_attention_decode_extras(void* stream, const void* qkv, int q_stride, void* out, const void* kv, float* part_o,
                                   float* part_ml, const int32_t* dec_items, int n_dec, const int32_t* item_start,
                                   const int32_t* item_end, const int32_t* table_off, const int32_t* block_ids, int hq,
                                   int hkv, int head_dim, int nsplit, float scale, int window, int min_split_keys,
-                                  int exact_weights, const float* sink, const float* dist_bias, int n_dist);
+                                  int exact_weights, const float* sink, const float* dist_bias, int n_dist,
+                            const void* gate, int64_t gate_row);
+
+// Attention with short convolutions, between the input product and the attention: rows of (hq + 2 hkv) heads of d
+// channels (in_row elements apart); every channel passes y[t] = sum_j taps_w[j][c] u[t - taps + 1 + j] (continued in front of an
+// item's first token from the inputs saved in its slot: state + slot * state_row, [taps - 1][channels], oldest first,
+// replaced by the item's last ones), q and k heads are divided by their root mean square over norm_dim (0: not), multiplied
+// by q_weight / k_weight (float [d] or NULL) and rotated (pairs (i, i + d/2), table [pos][d/2] or NULL). q goes to q_out
+// [tokens][hq * d], k and v to the pages (kv NULL: nowhere).
+int psamd_qkv_conv_append(void* stream, const void* in, int act_dtype, int64_t in_row, const float* taps_w, int taps, int hq, int hkv,
+                          int d, const int32_t* positions, const float* table, int norm_dim, float eps, const float* q_weight,
+                          const float* k_weight, void* q_out, void* kv, const int32_t* write_slot, float* state, int64_t state_row,
+                          const int32_t* tok_item, const int32_t* item_start, const int32_t* slots, int64_t tokens, int items);
+
+// Retention (linear attention with a fixed decay per head), gated and normalized per head: see retention.hip. rows: q, k
+// (heads of dim_p), v, gate (heads of vdim_p) at their columns; table float [pos][rot / 2][2]; powers float [heads]
+// [psamd_retention_powers()]: powers of the heads' decays from 0 on; state float, of slot s at state + s * state_row, [heads]
+// [dim_p][vdim_p]; pf_tiles / pf_blocks: the step's tiles of 32 tokens and runs of four of them; dec_items: its single-token
+// items; sums: room for n_blocks * heads * dim_p * vdim_p floats; out [tokens][heads * vdim_p].
+int psamd_retention_powers(void);
+int psamd_retention(void* stream, const void* rows, int act_dtype, int64_t row, int q_col, int k_col, int v_col, int g_col,
+                    const int32_t* positions, const float* table, int rot, const float* powers, float k_scale, float* state,
+                    int64_t state_row, const int32_t* item_start, const int32_t* slots, const int32_t* pf_tiles, int n_tiles,
+                    int tile_tokens, const int32_t* pf_blocks, int n_blocks, const int32_t* dec_items, int n_dec, float* sums,
+                    int heads, int dim_p, int vdim_p, int vdim, float eps, void* out);
+
+// residual[r] += norm(y[r]) * weight, norm(y) = y / sqrt(mean(y^2) + eps), y = a, or with b given y = scale *
+// (norm(a) * a_weight + norm(b) * b_weight) with in_eps inside; a and b are one tensor or float slices (stride elements
+// apart) that are summed first. out (or NULL): the new rows in out_dtype.
+int psamd_output_norm(void* stream, float* residual, const void* a, int a_dtype, int a_slices, int64_t a_stride, const float* a_weight,
+                      const void* b, int b_dtype, int b_slices, int64_t b_stride, const float* b_weight, float scale, float in_eps,
+                      const float* weight, float eps, void* out, int out_dtype, int64_t rows, int hidden);
+
+// out[t] = table[id] + bigram[(previous id * mul_prev + id * mul_cur) mod buckets], bigram[buckets] for a sequence's first
+// token; bigram [buckets + 1, hidden] in the table's dtype; copy (or NULL): the same rows in that dtype. state: int32,
+// of slot s at state + s * state_row: the item's last token + 1, 0 for none; read and replaced.
+int psamd_embed_bigram(void* stream, const int32_t* ids, const void* table, const void* bigram, int table_dtype, float* out, void* copy,
+                       int64_t tokens, int hidden, int vocab, int64_t buckets, int64_t mul_prev, int64_t mul_cur, int32_t* state,
+                       int64_t state_row, const int32_t* tok_item, const int32_t* item_start, const int32_t* slots);
 
 // out[r] = argmax (temperature[r] <= 0) or the inverse-CDF draw with uniform[r] in [0, 1).
 int64_t psamd_sample_scratch_floats(int rows);

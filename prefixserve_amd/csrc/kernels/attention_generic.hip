@@ -3,7 +3,8 @@
 // of heads and groups, optional sliding window, an optional
 // learned sink per head (a term exp(sink) in the softmax's denominator that has no key and no
 // value) and an optional bias on the scaled score that depends on the head and on how far back
-// the key lies (a table per head, its last entry standing for every larger distance).
+// the key lies (a table per head, its last entry standing for every larger distance), and an optional gate: output
+// (t, h, i) times sigmoid(gate[t, h, i]).
 // It is the attention of the exact 32-bit path and the fallback for shapes the
 // matrix-core kernels do not take.
 //
@@ -23,7 +24,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ tok_item,
     const int32_t* __restrict__ table_off, const int32_t* __restrict__ block_ids,
     int hq, int hkv, int d, float scale, int window, const float* __restrict__ sink,
-    const float* __restrict__ dist_bias, int n_dist) {
+    const float* __restrict__ dist_bias, int n_dist, const A* __restrict__ gate, int64_t gate_row) {
   __shared__ float q_s[kMaxHead];
   __shared__ float p_s[kWave];
   __shared__ int32_t base_s[kWave];   // element offset of (page, kv head) for each key of the chunk
@@ -89,7 +90,10 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
 #pragma unroll
   for (int dd = 0; dd < kMaxHead / kWave; ++dd) {
     const int i = lane + dd * kWave;
-    if (i < d) o[i] = from_float<A>(acc[dd] * inv);
+    if (i >= d) continue;
+    float y = acc[dd] * inv;
+    if (gate != nullptr) y *= 1.f / (1.f + expf(-to_float<A>(gate[t * gate_row + static_cast<int64_t>(h) * d + i])));
+    o[i] = from_float<A>(y);
   }
 }
 
@@ -193,7 +197,8 @@ extern "C" int psamd_attention_generic(void* stream, const void* qkv, int q_stri
                                        int act_dtype, int64_t tokens, const int32_t* positions,
                                        const int32_t* tok_item, const int32_t* table_off, const int32_t* block_ids,
                                        int hq, int hkv, int head_dim, float scale, int window, const float* sink,
-                                       const float* dist_bias, int n_dist) {
+                                       const float* dist_bias, int n_dist, const void* gate, int64_t gate_row) {
+  PSAMD_REQUIRE(gate == nullptr || gate_row >= static_cast<int64_t>(hq) * head_dim, "the gate's rows");
   PSAMD_REQUIRE(dist_bias == nullptr || n_dist >= 1, "a distance bias needs at least one entry per head");
   PSAMD_REQUIRE(tokens >= 0 && hq > 0 && hkv > 0 && hq % hkv == 0, "bad head counts");
   PSAMD_REQUIRE(head_dim > 0 && head_dim <= kMaxHead, "head_dim must be in [1, 1024]");
@@ -204,11 +209,13 @@ extern "C" int psamd_attention_generic(void* stream, const void* qkv, int q_stri
   if (act_dtype == kBF16) {
     attention_generic_kernel<bf16_t><<<grid, dim3(64), 0, s>>>(
         static_cast<const bf16_t*>(qkv), q_stride, static_cast<bf16_t*>(out), static_cast<const bf16_t*>(kv),
-        positions, tok_item, table_off, block_ids, hq, hkv, head_dim, scale, window, sink, dist_bias, n_dist);
+        positions, tok_item, table_off, block_ids, hq, hkv, head_dim, scale, window, sink, dist_bias, n_dist,
+        static_cast<const bf16_t*>(gate), gate_row);
   } else if (act_dtype == kF32) {
     attention_generic_kernel<float><<<grid, dim3(64), 0, s>>>(
         static_cast<const float*>(qkv), q_stride, static_cast<float*>(out), static_cast<const float*>(kv),
-        positions, tok_item, table_off, block_ids, hq, hkv, head_dim, scale, window, sink, dist_bias, n_dist);
+        positions, tok_item, table_off, block_ids, hq, hkv, head_dim, scale, window, sink, dist_bias, n_dist,
+        static_cast<const float*>(gate), gate_row);
   } else {
     return fail("psamd_attention_generic: activation dtype must be float32 or bfloat16");
   }

@@ -32,14 +32,25 @@ typedef __attribute__((ext_vector_type(16))) float f32x16;
 
 // What a softmax may have beyond keys: a learned sink per head (exp(sink[h]) joins the denominator;
 // it has no key and no value) and a bias on the scaled score that depends on the head and on how
-// far back the key lies, bias[h][min(i - j, n_dist - 1)]. Either pointer may be null. The entry
+// far back the key lies, bias[h][min(i - j, n_dist - 1)]; and a gate on what leaves it, entry by entry:
+// output (t, h, d) times sigmoid(gate[t * gate_row + h * D + d]). Any pointer may be null. The entry
 // points with these arguments set g_extras for the launches they make.
 struct Extras {
   const float* sink;
   const float* bias;
   int n_dist;
+  const bf16_t* gate;
+  int64_t gate_row;
 };
-static thread_local Extras g_extras = {nullptr, nullptr, 0};
+constexpr Extras kNoExtras = {nullptr, nullptr, 0, nullptr, 0};
+static thread_local Extras g_extras = kNoExtras;
+
+// The gate's factors for outputs d .. d + 3 of head h of token t.
+__device__ __forceinline__ float4 gate4(const Extras& ex, int64_t t, int64_t at) {
+  const uint2 q = *reinterpret_cast<const uint2*>(ex.gate + t * ex.gate_row + at);
+  return float4{1.f / (1.f + __expf(-__uint_as_float(q.x << 16))), 1.f / (1.f + __expf(-__uint_as_float(q.x & 0xffff0000u))),
+                1.f / (1.f + __expf(-__uint_as_float(q.y << 16))), 1.f / (1.f + __expf(-__uint_as_float(q.y & 0xffff0000u)))};
+}
 constexpr float kLog2e = 1.44269504088896340736f;
 // A 16-byte piece in registers. A plain vector: HIP's uint4 is a struct, and copies of it in
 // arrays were compiled to copies through scratch memory.
@@ -363,6 +374,10 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
             *reinterpret_cast<float4*>(part_o + part_slot * D + d) =
                 float4{r[4 * v4 + 0], r[4 * v4 + 1], r[4 * v4 + 2], r[4 * v4 + 3]};
           } else if (d < D) {
+            if (ex.gate != nullptr) {
+              const float4 f = gate4(ex, t0 + qi, h * D + d);
+              r[4 * v4 + 0] *= f.x; r[4 * v4 + 1] *= f.y; r[4 * v4 + 2] *= f.z; r[4 * v4 + 3] *= f.w;
+            }
             ushort4 pk;
             pk.x = float_to_bf16(r[4 * v4 + 0] * inv);
             pk.y = float_to_bf16(r[4 * v4 + 1] * inv);
@@ -397,7 +412,7 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_kernel(
     const int32_t* __restrict__ pool_block_ids, int block, const float* __restrict__ gate) {
   float* part_o = nullptr;
   float* part_ml = nullptr;
-  const Extras ex = {nullptr, nullptr, 0};
+  const Extras ex = kNoExtras;
   constexpr int D = 16 * NS;
   constexpr int DT = (D + 31) / 32;
   constexpr int DTC = DT < 2 ? DT : 2;      // d-tiles merged per pass (bounds the LDS buffer)
@@ -1051,11 +1066,16 @@ __global__ __launch_bounds__(256 * KP, NS <= 4 ? 4 : 2) void attn_prefill_groupe
     for (int v4 = 0; v4 < 4; ++v4) {
       const int d = 32 * dt + 8 * v4 + 4 * hi;
       if (d < D) {
+        float4 f = {inv, inv, inv, inv};
+        if (ex.gate != nullptr) {
+          const float4 gt = gate4(ex, t0 + qi, h * D + d);
+          f = float4{inv * gt.x, inv * gt.y, inv * gt.z, inv * gt.w};
+        }
         ushort4 pk;
-        pk.x = float_to_bf16(o[dt][4 * v4 + 0] * inv);
-        pk.y = float_to_bf16(o[dt][4 * v4 + 1] * inv);
-        pk.z = float_to_bf16(o[dt][4 * v4 + 2] * inv);
-        pk.w = float_to_bf16(o[dt][4 * v4 + 3] * inv);
+        pk.x = float_to_bf16(o[dt][4 * v4 + 0] * f.x);
+        pk.y = float_to_bf16(o[dt][4 * v4 + 1] * f.y);
+        pk.z = float_to_bf16(o[dt][4 * v4 + 2] * f.z);
+        pk.w = float_to_bf16(o[dt][4 * v4 + 3] * f.w);
         *reinterpret_cast<ushort4*>(op + d) = pk;
       }
     }
@@ -1112,6 +1132,10 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(
   }
   if (ex.sink != nullptr) ll += __builtin_amdgcn_exp2f(ex.sink[h] * kLog2e - mm);
   const float inv = 1.f / ll;
+  if (ex.gate != nullptr) {
+    const float4 f = gate4(ex, t0 + q, static_cast<int64_t>(h) * d + 4 * chunk);
+    acc.x *= f.x; acc.y *= f.y; acc.z *= f.z; acc.w *= f.w;
+  }
   ushort4 pk;
   pk.x = float_to_bf16(acc.x * inv);
   pk.y = float_to_bf16(acc.y * inv);
@@ -1336,7 +1360,9 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     }
     if (nsplit == 1) {   // nothing to merge with: this is the result
       if (ex.sink != nullptr) ll += __expf(ex.sink[kvh * group + hh] - mm);
-      out[t * (static_cast<int64_t>(hq) * D) + static_cast<int64_t>(kvh * group + hh) * D + d] = float_to_bf16(acc / ll);
+      const int64_t at = static_cast<int64_t>(kvh * group + hh) * D + d;
+      if (ex.gate != nullptr) acc *= 1.f / (1.f + __expf(-bf16_to_float(ex.gate[t * ex.gate_row + at])));
+      out[t * (static_cast<int64_t>(hq) * D) + at] = float_to_bf16(acc / ll);
       continue;
     }
     const int64_t slot = (static_cast<int64_t>(di) * hq + kvh * group + hh) * nsplit + split;
@@ -1383,6 +1409,7 @@ __global__ __launch_bounds__(64) void attn_decode_merge_kernel(
     }
 #pragma unroll 8
     for (int s = s0; s < nsplit; ++s) acc += wgt_s[s] * part_o[(base + s) * d + i];
+    if (ex.gate != nullptr) acc *= 1.f / (1.f + __expf(-bf16_to_float(ex.gate[t * ex.gate_row + h * d + i])));
     out[t * (static_cast<int64_t>(hq) * d) + h * d + i] = float_to_bf16(acc);
   }
 }
@@ -1812,19 +1839,22 @@ int psamd_attention_decode(void* stream, const void* qkv, int q_stride, void* ou
 }
 
 // The two entry points above with a softmax that has more than keys: sink (float [hq] or NULL) and
-// dist_bias (float [hq, n_dist] or NULL), see psamd_attention_generic.
+// dist_bias (float [hq, n_dist] or NULL), and a gate on the output (bfloat16 rows, gate_row elements apart, or
+// NULL), see psamd_attention_generic.
 int psamd_attention_prefill_extras(void* stream, const void* qkv, int q_stride, void* out, const void* kv,
                                    const int32_t* pf_tiles, int n_tiles, const int32_t* pf_blocks, int n_blocks,
                                    int max_kv_len, const int32_t* item_start, const int32_t* item_pos0,
                                    const int32_t* table_off, const int32_t* block_ids, int hq, int hkv, int head_dim,
                                    float scale, int window, float* part_o, float* part_ml, int nsplit, int exact_weights,
-                                   const float* sink, const float* dist_bias, int n_dist) {
+                                   const float* sink, const float* dist_bias, int n_dist, const void* gate, int64_t gate_row) {
   PSAMD_REQUIRE(dist_bias == nullptr || (n_dist >= 1 && scale != 0.f), "a distance bias needs entries and a scale that is not zero");
-  g_extras = Extras{sink, dist_bias, n_dist};
+  PSAMD_REQUIRE(gate == nullptr || (gate_row % 4 == 0 && gate_row >= static_cast<int64_t>(hq) * head_dim &&
+                                    reinterpret_cast<uintptr_t>(gate) % 8 == 0), "the gate's rows");
+  g_extras = Extras{sink, dist_bias, n_dist, static_cast<const bf16_t*>(gate), gate_row};
   const int rc = psamd_attention_prefill(stream, qkv, q_stride, out, kv, pf_tiles, n_tiles, pf_blocks, n_blocks, max_kv_len,
                                          item_start, item_pos0, table_off, block_ids, hq, hkv, head_dim, scale, window,
                                          part_o, part_ml, nsplit, exact_weights);
-  g_extras = Extras{nullptr, nullptr, 0};
+  g_extras = kNoExtras;
   return rc;
 }
 
@@ -1832,13 +1862,15 @@ int psamd_attention_decode_extras(void* stream, const void* qkv, int q_stride, v
                                   float* part_ml, const int32_t* dec_items, int n_dec, const int32_t* item_start,
                                   const int32_t* item_end, const int32_t* table_off, const int32_t* block_ids, int hq,
                                   int hkv, int head_dim, int nsplit, float scale, int window, int min_split_keys,
-                                  int exact_weights, const float* sink, const float* dist_bias, int n_dist) {
+                                  int exact_weights, const float* sink, const float* dist_bias, int n_dist, const void* gate, int64_t gate_row) {
   PSAMD_REQUIRE(dist_bias == nullptr || n_dist >= 1, "a distance bias needs at least one entry per head");
-  g_extras = Extras{sink, dist_bias, n_dist};
+  PSAMD_REQUIRE(gate == nullptr || (gate_row % 4 == 0 && gate_row >= static_cast<int64_t>(hq) * head_dim &&
+                                    reinterpret_cast<uintptr_t>(gate) % 8 == 0), "the gate's rows");
+  g_extras = Extras{sink, dist_bias, n_dist, static_cast<const bf16_t*>(gate), gate_row};
   const int rc = psamd_attention_decode(stream, qkv, q_stride, out, kv, part_o, part_ml, dec_items, n_dec, item_start,
                                         item_end, table_off, block_ids, hq, hkv, head_dim, nsplit, scale, window,
                                         min_split_keys, exact_weights);
-  g_extras = Extras{nullptr, nullptr, 0};
+  g_extras = kNoExtras;
   return rc;
 }
 

@@ -10,16 +10,20 @@
 //
 // Router: z = x . w_r[e] (+ bias[e]) in float; the `top` largest are taken, the lower index among
 // equals. mode 0: the score is sigmoid(z) and is the weight as it is; mode 1: the weights are the
-// softmax over the chosen z alone. Expert: with h = weight * x, g = min(gate h, limit), u = clamp(up h,
+// softmax over the chosen z alone; mode 2: the score is the softmax over all z, the choice goes by score +
+// correction[e] (which may be negative) and the weight is the score as it is. Expert: with h = weight * x, g = min(gate h, limit), u = clamp(up h,
 // -limit, limit), act = g * sigmoid(gate_alpha * g) * (u + up_shift), out = down act. There the weight
 // multiplies the expert's input, so it cannot be pulled out of the clamps; with weight_on_output the
 // expert sees x itself and the weight multiplies out (limit = infinity, gate_alpha = 1, up_shift = 0
 // then make the plain SiLU-gated expert). The other kind of expert has no gate: act = max(up h, 0)^2
 // (kExpertSquaredRelu), its first matrix is [F, K].
 //
-// With groups (mode 0): the experts form `groups` equal runs of neighbours, a run's score is the sum of its
-// two largest scores, and only experts of the `keep` best runs (the lower index among equals) can be
-// chosen. The weights are multiplied by `factor`.
+// With groups (modes 0 and 2): the experts form `groups` equal runs of neighbours, a run's score is the sum of its
+// two largest scores (group_max: its largest), each with its correction, and only experts of the `keep` best runs
+// (the lower index among equals) can be chosen. The weights are multiplied by `factor`.
+//
+// Choices from `experts` on are identity experts: they have no matrices, their output is the token itself times the
+// weight. The grouped form lists their pairs behind the experts' and lets the second product's launch copy them.
 //
 // `out` is float slices [top][tokens][K], or, for a small bfloat16 step, the float residual stream itself
 // (`into_stream`): every pair then adds col_scale[k] * weight * value with float atomics, and nobody adds
@@ -44,6 +48,8 @@ struct RouterRule {
   int groups;
   int keep;
   float factor;
+  int group_max;
+  const float* correction;             // mode 2: [experts] or null
 };
 
 // dst += v at the memory side, nothing returned.
@@ -104,7 +110,8 @@ __device__ __forceinline__ void wave_best(float& best, int& at) {
 
 // Takes the experts outside the best groups out of the choice: their entries of score[] (LDS) become kTaken.
 // Lane l holds the scores of groups l, l + 64, ... (at most kMaxRouterGroups in all).
-__device__ __forceinline__ void keep_best_groups(float* score, int experts, int groups, int keep, int lane) {
+__device__ __forceinline__ void keep_best_groups(float* score, int experts, const RouterRule& rule, int lane) {
+  const int groups = rule.groups, keep = rule.keep;
   constexpr int kPer = kMaxRouterGroups / kWave;
   const float kTaken = -__builtin_inff();
   const int size = experts / groups;
@@ -118,7 +125,7 @@ __device__ __forceinline__ void keep_best_groups(float* score, int experts, int 
     if (grp < groups) {
       float a = kTaken, b = 0.f;                          // the two largest; a group of one expert has one
       for (int e = grp * size; e < (grp + 1) * size; ++e) {
-        const float s = score[e];
+        const float s = rule.correction != nullptr ? score[e] + rule.correction[e] : score[e];
         if (s > a) {
           b = a == kTaken ? 0.f : a;
           a = s;
@@ -126,7 +133,7 @@ __device__ __forceinline__ void keep_best_groups(float* score, int experts, int 
           b = s;
         }
       }
-      sum[i] = a + b;
+      sum[i] = rule.group_max ? a : a + b;
     }
   }
   for (int j = 0; j < keep; ++j) {
@@ -159,6 +166,13 @@ __device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top,
   const float kTaken = -__builtin_inff();
   auto of = [](float v, int from) { return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), from)); };
   if (lane >= experts) s = kTaken;
+  float w = s;
+  if (rule.mode == 2) {
+    const float m = wave_max(s);                          // by all lanes: the moves between lanes need every one of them
+    const float p = lane < experts ? expf(s - m) : 0.f;
+    w = p / wave_sum(p);
+    s = lane >= experts ? kTaken : rule.correction != nullptr ? w + rule.correction[lane] : w;
+  }
   if (rule.groups > 0) {
     const int size = experts / rule.groups, mine = lane / size;
     float a = kTaken, b = kTaken;                         // the two largest of the lane's own group
@@ -170,7 +184,7 @@ __device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top,
           a = fmaxf(a, v);
         }
       }
-    const float sum = a + (size > 1 ? b : 0.f);
+    const float sum = rule.group_max ? a : a + (size > 1 ? b : 0.f);
     int ahead = 0;                                        // groups in front of the lane's own
     for (int grp = 0; grp < rule.groups; ++grp) {
       const float v = of(sum, grp * size);
@@ -184,7 +198,7 @@ __device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top,
     rank += (v > s || (v == s && e < lane)) ? 1 : 0;
   }
   const bool taken = lane < experts && rank < top && s > kTaken;
-  float w = s;
+  if (rule.mode == 0) w = s;
   if (rule.mode == 1) {
     const float m = wave_max(taken ? s : kTaken);
     // Summed in the order of the choice, largest first.
@@ -202,8 +216,8 @@ __device__ __forceinline__ void pick_top_in_lanes(float s, int experts, int top,
 }
 
 // The router's choice for one token by one wave: score[] (LDS, `experts` entries: sigmoid(z) in mode
-// 0, z in mode 1) -> chosen / weight [top], largest first, the lower index among equals; taken
-// entries are overwritten. Mode 1 then turns the chosen z into their softmax.
+// 0, z in modes 1 and 2) -> chosen / weight [top], largest first, the lower index among equals; taken
+// entries are overwritten. Mode 1 then turns the chosen z into their softmax; mode 2 turns all z into their softmax first.
 __device__ __forceinline__ void pick_top(float* score, int experts, int top, RouterRule rule, int32_t* __restrict__ chosen,
                                          float* __restrict__ weight, int lane) {
   const float kTaken = -__builtin_inff();
@@ -211,12 +225,25 @@ __device__ __forceinline__ void pick_top(float* score, int experts, int top, Rou
     pick_top_in_lanes(lane < experts ? score[lane] : 0.f, experts, top, rule, chosen, weight, lane);
     return;
   }
-  if (rule.groups > 0) keep_best_groups(score, experts, rule.groups, rule.keep, lane);
+  if (rule.mode == 2) {
+    float m = kTaken, sum = 0.f;
+    for (int e = lane; e < experts; e += kWave) m = fmaxf(m, score[e]);
+    m = wave_max(m);
+    for (int e = lane; e < experts; e += kWave) {
+      score[e] = expf(score[e] - m);
+      sum += score[e];
+    }
+    sum = wave_sum(sum);
+    for (int e = lane; e < experts; e += kWave) score[e] /= sum;
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+  }
+  if (rule.groups > 0) keep_best_groups(score, experts, rule, lane);
   for (int j = 0; j < top; ++j) {
     float best = kTaken;
     int at = 0x7fffffff;
     for (int e = lane; e < experts; e += kWave) {
-      const float s = score[e];
+      const float s = rule.correction != nullptr ? score[e] + rule.correction[e] : score[e];
       if (s > best) {                                    // ascending e: the first of equals stays
         best = s;
         at = e;
@@ -225,7 +252,7 @@ __device__ __forceinline__ void pick_top(float* score, int experts, int top, Rou
     wave_best(best, at);
     if (lane == 0) {
       chosen[j] = at;
-      weight[j] = rule.mode == 0 ? rule.factor * best : best;
+      weight[j] = rule.mode == 0 ? rule.factor * best : rule.mode == 2 ? (at != 0x7fffffff ? rule.factor * score[at] : 0.f) : best;
       if (at != 0x7fffffff) score[at] = kTaken;
     }
     __builtin_amdgcn_wave_barrier();
@@ -300,7 +327,8 @@ __global__ __launch_bounds__(256) void moe_gate_up_rows_kernel(
   const int64_t pair = blockIdx.x;
   const int64_t t = pair / top;
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x >> 6;
-  const int e = min(max(chosen[pair], 0), experts - 1);
+  if (chosen[pair] >= experts) return;                   // an identity expert has no activations
+  const int e = max(chosen[pair], 0);
   const float wgt = weight_on_output ? 1.f : weight[pair];
   for (int i = threadIdx.x; i < K; i += blockDim.x) rows_smem[i] = wgt * to_float<A>(x[t * K + i]);
   __syncthreads();
@@ -327,13 +355,21 @@ template <typename A>
 __global__ __launch_bounds__(256) void moe_down_rows_kernel(
     const A* __restrict__ act, const int32_t* __restrict__ chosen, const A* __restrict__ w_down,
     float* __restrict__ out, int64_t tokens, int K, int F, int experts, int top, const float* __restrict__ out_weight,
-    int into_stream, const float* __restrict__ col_scale) {
+    int into_stream, const float* __restrict__ col_scale, const A* __restrict__ x, const float* __restrict__ weight) {
   extern __shared__ __align__(16) float rows_smem[];     // act[F]
   const int64_t pair = blockIdx.x;
   const int64_t t = pair / top;
   const int j = static_cast<int>(pair - t * top);
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x >> 6;
-  const int e = min(max(chosen[pair], 0), experts - 1);
+  if (chosen[pair] >= experts) {                         // an identity expert: the token itself
+    const int k = static_cast<int>(blockIdx.y) * kRowsPerBlock + threadIdx.x;
+    if (threadIdx.x >= kRowsPerBlock || k >= K) return;
+    const float y = weight[pair] * to_float<A>(x[t * K + k]);
+    if (into_stream) add_float(out + t * K + k, col_scale != nullptr ? col_scale[k] * y : y);
+    else out[(static_cast<int64_t>(j) * tokens + t) * K + k] = y;
+    return;
+  }
+  const int e = max(chosen[pair], 0);
   for (int i = threadIdx.x; i < F; i += blockDim.x) rows_smem[i] = to_float<A>(act[pair * F + i]);
   __syncthreads();
   const A* we = w_down + static_cast<int64_t>(e) * K * F;
@@ -420,7 +456,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* __restri
 // The choice from logits and the sorting in one workgroup of 16 waves, for steps of so few tokens
 // that one workgroup does the choice at once (a decode step): a wave per token, then the sorting above.
 __global__ __launch_bounds__(1024) void moe_topk_group_kernel(const float* __restrict__ z, int32_t* __restrict__ chosen,
-                                                              float* __restrict__ weight, int tokens, int experts, int top,
+                                                              float* __restrict__ weight, int tokens, int experts, int buckets, int top,
                                                               int tile_rows, int max_tiles, int32_t* __restrict__ sorted,
                                                               int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_first,
                                                               int32_t* __restrict__ tile_count, const float* __restrict__ bias,
@@ -436,7 +472,7 @@ __global__ __launch_bounds__(1024) void moe_topk_group_kernel(const float* __res
   }
   __threadfence_block();
   __syncthreads();                             // the workgroup's own writes of `chosen` are read below
-  group_pairs(chosen, tokens * top, experts, tile_rows, max_tiles, sorted, tile_expert, tile_first, tile_count, group_smem,
+  group_pairs(chosen, tokens * top, buckets, tile_rows, max_tiles, sorted, tile_expert, tile_first, tile_count, group_smem,
               group_smem + experts, group_smem + 2 * experts, group_smem + 3 * experts, group_smem + 4 * experts);
 }
 
@@ -464,7 +500,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const int32_t* __restrict__ sorted, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_first,
     const int32_t* __restrict__ tile_count, bf16_t* __restrict__ out_act, float* __restrict__ out_f32, int64_t tokens,
     int K, int N, int top, float gate_alpha, float limit, float up_shift, int into_stream,
-    const float* __restrict__ col_scale) {
+    const float* __restrict__ col_scale, int experts, const bf16_t* __restrict__ x, const float* __restrict__ weight) {
   constexpr bool GATED = FORM == kFormGated;
   constexpr int kGroupBK = group_bk(MT);
   constexpr int kGroupLD = kGroupBK + 8;                     // LDS row stride of the staged pairs, in elements
@@ -478,6 +514,19 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
   const int e = tile_expert[slot];
   if (e < 0) return;                            // uniform for the workgroup
   const int first = tile_first[slot], count = tile_count[slot];
+  if (e >= experts) {                           // a tile of identity pairs: the tokens themselves times their weights
+    if (FORM != kFormDown) return;
+    constexpr int COLS = 64 * RT;
+    for (int idx = threadIdx.x; idx < count * COLS; idx += 256) {
+      const int pair = sorted[first + idx / COLS], n = static_cast<int>(blockIdx.x) * COLS + idx % COLS;
+      if (n >= N) continue;
+      const int64_t t = pair / top;
+      const float y = weight[pair] * bf16_to_float(x[t * N + n]);
+      if (into_stream) add_float(out_f32 + t * N + n, col_scale != nullptr ? col_scale[n] * y : y);
+      else out_f32[(static_cast<int64_t>(pair % top) * tokens + t) * N + n] = y;
+    }
+    return;
+  }
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int r = lane & 15, g = lane >> 4;
   const int n0 = (static_cast<int>(blockIdx.x) * 4 + wave) * 16 * RT;     // this wave's first column
@@ -634,7 +683,7 @@ struct ExpertCall {
   void* act;
   float* out;
   int64_t tokens;
-  int K, F, experts, top, kind;
+  int K, F, experts, top, kind;        // experts: those with matrices
   float gate_alpha, limit, up_shift;
   int weight_on_output, into_stream;
   const float* col_scale;
@@ -652,7 +701,8 @@ static void run_grouped(hipStream_t s, const ExpertCall& c, const int32_t* ints,
   moe_grouped_kernel<MT, RT, FORM><<<grid, dim3(256), 0, s>>>(
       static_cast<const bf16_t*>(down ? c.act : c.x), (c.weight_on_output != 0) == down ? c.weight : nullptr,
       static_cast<const bf16_t*>(down ? c.w_down : c.w_in), sorted, t_e, t_f, t_c, down ? nullptr : static_cast<bf16_t*>(c.act),
-      down ? c.out : nullptr, c.tokens, K, N, c.top, c.gate_alpha, c.limit, c.up_shift, c.into_stream, c.col_scale);
+      down ? c.out : nullptr, c.tokens, K, N, c.top, c.gate_alpha, c.limit, c.up_shift, c.into_stream, c.col_scale, c.experts,
+      static_cast<const bf16_t*>(c.x), c.weight);
 }
 
 template <int MT, int RT>
@@ -675,17 +725,18 @@ static int launch_experts_rows(hipStream_t s, const ExpertCall& c) {
   moe_down_rows_kernel<A><<<dim3(pairs, static_cast<unsigned>(ceil_div(c.K, kRowsPerBlock))), dim3(256),
                             sizeof(float) * c.F, s>>>(
       static_cast<const A*>(c.act), c.chosen, static_cast<const A*>(c.w_down), c.out, c.tokens, c.K, c.F, c.experts, c.top,
-      c.weight_on_output ? c.weight : nullptr, c.into_stream, c.col_scale);
+      c.weight_on_output ? c.weight : nullptr, c.into_stream, c.col_scale, static_cast<const A*>(c.x), c.weight);
   return check_launch("psamd_moe_experts_rows (down)");
 }
 
 // The rule as the entry points take it, checked on the host.
-static const char* bad_rule(int mode, int groups, int keep, int experts, int top) {
-  if (mode != 0 && mode != 1) return "router mode 0 (sigmoid scores) or 1 (softmax over the chosen)";
-  if (groups == 0) return nullptr;
-  if (mode != 0) return "groups of experts go with sigmoid scores";
-  if (groups < 1 || groups > kMaxRouterGroups || experts % groups != 0) return "the experts must form at most 256 equal groups";
-  if (keep < 1 || keep > groups || top > keep * (experts / groups)) return "the kept groups hold fewer experts than are chosen";
+static const char* bad_rule(const RouterRule& r, int experts, int top) {
+  if (r.mode < 0 || r.mode > 2) return "router mode 0 (sigmoid scores), 1 (softmax over the chosen) or 2 (softmax over all)";
+  if (r.correction != nullptr && r.mode != 2) return "a correction of the choice goes with the softmax over all experts";
+  if (r.groups == 0) return nullptr;
+  if (r.mode == 1) return "groups of experts go with scores that do not depend on the choice";
+  if (r.groups < 1 || r.groups > kMaxRouterGroups || experts % r.groups != 0) return "the experts must form at most 256 equal groups";
+  if (r.keep < 1 || r.keep > r.groups || top > r.keep * (experts / r.groups)) return "the kept groups hold fewer experts than are chosen";
   return nullptr;
 }
 
@@ -714,10 +765,10 @@ int psamd_moe_grouped_max_tiles(int64_t pairs, int experts);
 
 int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_router, int32_t* chosen, float* weight,
                     int64_t tokens, int K, int experts, int top, const float* bias, int mode,
-                    int groups, int keep, float factor) {
+                    int groups, int keep, float factor, int group_max, const float* correction) {
   PSAMD_REQUIRE(tokens >= 0 && K > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
-  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
-  const RouterRule rule{mode, groups, keep, factor};
+  const RouterRule rule{mode, groups, keep, factor, group_max, correction};
+  if (const char* bad = bad_rule(rule, experts, top)) return fail(bad);
   PSAMD_REQUIRE(sizeof(float) * (static_cast<size_t>(K) + experts) <= 64 * 1024, "row and scores do not fit in LDS");
   PSAMD_REQUIRE(tokens <= 2147483647LL, "too many tokens for one launch");
   if (tokens == 0) return 0;
@@ -738,10 +789,10 @@ int psamd_moe_route(void* stream, const void* x, int x_dtype, const float* w_rou
 
 int psamd_moe_topk(void* stream, const float* logits, int32_t* chosen, float* weight, int64_t tokens, int experts,
                    int top, const float* bias, int mode,
-                   int groups, int keep, float factor) {
+                   int groups, int keep, float factor, int group_max, const float* correction) {
   PSAMD_REQUIRE(tokens >= 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
-  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
-  const RouterRule rule{mode, groups, keep, factor};
+  const RouterRule rule{mode, groups, keep, factor, group_max, correction};
+  if (const char* bad = bad_rule(rule, experts, top)) return fail(bad);
   PSAMD_REQUIRE(sizeof(float) * 4 * static_cast<size_t>(experts) <= 64 * 1024, "scores do not fit in LDS");
   PSAMD_REQUIRE(ceil_div(tokens, 4) <= 2147483647LL, "too many tokens for one launch");
   if (tokens == 0) return 0;
@@ -751,17 +802,17 @@ int psamd_moe_topk(void* stream, const float* logits, int32_t* chosen, float* we
 }
 
 int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, float* weight, int32_t* ints, int64_t tokens,
-                         int experts, int top, const float* bias, int mode,
-                         int groups, int keep, float factor) {
+                         int experts, int buckets, int top, const float* bias, int mode,
+                         int groups, int keep, float factor, int group_max, const float* correction) {
   PSAMD_REQUIRE(tokens >= 1 && tokens <= 64 && experts > 0 && experts <= 1024 && top >= 1 && top <= experts, "bad sizes");
-  if (const char* bad = bad_rule(mode, groups, keep, experts, top)) return fail(bad);
-  const RouterRule rule{mode, groups, keep, factor};
-  PSAMD_REQUIRE(ints != nullptr, "the grouping needs its integer scratch");
+  const RouterRule rule{mode, groups, keep, factor, group_max, correction};
+  if (const char* bad = bad_rule(rule, experts, top)) return fail(bad);
+  PSAMD_REQUIRE(ints != nullptr && buckets >= 1 && buckets <= experts, "the grouping needs its integer scratch, and buckets for the experts");
   const int64_t pairs = tokens * top;
-  const int rows = psamd_moe_grouped_tile_rows(pairs, experts);
-  const int max_tiles = psamd_moe_grouped_max_tiles(pairs, experts);
+  const int rows = psamd_moe_grouped_tile_rows(pairs, buckets);
+  const int max_tiles = psamd_moe_grouped_max_tiles(pairs, buckets);
   moe_topk_group_kernel<<<dim3(1), dim3(1024), sizeof(int32_t) * (4 * experts + 1) + sizeof(float) * 16 * experts,
-                          static_cast<hipStream_t>(stream)>>>(logits, chosen, weight, static_cast<int>(tokens), experts, top, rows,
+                          static_cast<hipStream_t>(stream)>>>(logits, chosen, weight, static_cast<int>(tokens), experts, buckets, top, rows,
                                                               max_tiles, ints, ints + pairs, ints + pairs + max_tiles,
                                                               ints + pairs + 2 * max_tiles, bias, rule);
   return check_launch("psamd_moe_topk_group");
@@ -769,9 +820,9 @@ int psamd_moe_topk_group(void* stream, const float* logits, int32_t* chosen, flo
 
 int psamd_moe_experts_rows(void* stream, const void* x, const int32_t* chosen, const float* weight,
                            const void* w_in, const void* w_down, void* act, float* out, int dtype,
-                           int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
+                           int64_t tokens, int K, int F, int experts, int identity, int top, float gate_alpha, float limit,
                            float up_shift, int weight_on_output, int kind, int into_stream, const float* col_scale) {
-  PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
+  PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && identity >= 0 && top >= 1 && top <= experts + identity, "bad sizes");
   PSAMD_REQUIRE(kind == kExpertGated || kind == kExpertSquaredRelu, "experts are gated (0) or squared ReLU without a gate (1)");
   PSAMD_REQUIRE(sizeof(float) * static_cast<size_t>(std::max(K, F)) <= 64 * 1024, "a row does not fit in LDS");
   PSAMD_REQUIRE(tokens * top <= 2147483647LL && ceil_div(std::max(K, F), kRowsPerBlock) <= 65535, "too large for one launch");
@@ -800,23 +851,24 @@ int psamd_moe_grouped_max_tiles(int64_t pairs, int experts) {
 
 int psamd_moe_experts_grouped(void* stream, const void* x, const int32_t* chosen, const float* weight,
                               const void* w_in, const void* w_down, void* act, float* out, int32_t* ints,
-                              int64_t tokens, int K, int F, int experts, int top, float gate_alpha, float limit,
+                              int64_t tokens, int K, int F, int experts, int identity, int top, float gate_alpha, float limit,
                               float up_shift, int grouped_already, int weight_on_output, int kind, int into_stream,
                               const float* col_scale) {
   PSAMD_REQUIRE(kind == kExpertGated || kind == kExpertSquaredRelu, "experts are gated (0) or squared ReLU without a gate (1)");
-  PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && top >= 1 && top <= experts, "bad sizes");
+  PSAMD_REQUIRE(tokens >= 0 && K > 0 && F > 0 && experts > 0 && identity >= 0 && top >= 1 && top <= experts + identity, "bad sizes");
   PSAMD_REQUIRE(K % 8 == 0 && F % 8 == 0, "K and F must be multiples of 8");
   PSAMD_REQUIRE(experts <= 4096 && tokens * top <= (1 << 24), "too many experts or pairs");
   PSAMD_REQUIRE(ints != nullptr, "the grouping needs its integer scratch");
   if (tokens == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int64_t pairs = tokens * top;
-  const int rows = psamd_moe_grouped_tile_rows(pairs, experts);
-  const int max_tiles = psamd_moe_grouped_max_tiles(pairs, experts);
+  const int buckets = experts + (identity > 0 ? 1 : 0);      // all identity pairs lie in one, behind the experts'
+  const int rows = psamd_moe_grouped_tile_rows(pairs, buckets);
+  const int max_tiles = psamd_moe_grouped_max_tiles(pairs, buckets);
   PSAMD_REQUIRE(max_tiles <= 65535, "too many tiles for one launch");
   if (grouped_already == 0) {
-    moe_group_kernel<<<dim3(1), dim3(1024), sizeof(int32_t) * (4 * experts + 1), s>>>(
-        chosen, static_cast<int>(pairs), experts, rows, max_tiles, ints, ints + pairs, ints + pairs + max_tiles,
+    moe_group_kernel<<<dim3(1), dim3(1024), sizeof(int32_t) * (4 * buckets + 1), s>>>(
+        chosen, static_cast<int>(pairs), buckets, rows, max_tiles, ints, ints + pairs, ints + pairs + max_tiles,
         ints + pairs + 2 * max_tiles);
     if (check_launch("psamd_moe_experts_grouped (grouping)")) return 1;
   }

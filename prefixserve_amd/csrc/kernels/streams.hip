@@ -125,12 +125,13 @@ __global__ __launch_bounds__(256) void weighted_sum_kernel(const void* __restric
   out[e] = fmaf(a_scale, delta_at(a, a_dtype, a_slices, a_stride, e), b_scale * delta_at(b, b_dtype, b_slices, b_stride, e));
 }
 
-// kind 0 = GELU (exact), 1 = GELU (tanh form), 2 = SiLU, 3 = ReLU.
+// kind 0 = GELU (exact), 1 = GELU (tanh form), 2 = SiLU, 3 = ReLU, 4 = the square of ReLU.
 __device__ __forceinline__ float activate(float z, int kind) {
   if (kind == 0) return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
   if (kind == 1) return gelu_tanh_f(z);
   if (kind == 2) return z * sigmoid_f(z);
-  return fmaxf(z, 0.f);
+  z = fmaxf(z, 0.f);
+  return kind == 4 ? z * z : z;
 }
 
 // Sixteen bytes per thread and access (8 bfloat16 or 4 floats); the entries behind the last whole group one by one.
@@ -404,7 +405,7 @@ int psamd_weighted_sum(void* stream, const void* a, int a_dtype, int a_slices, i
 }
 
 int psamd_activation(void* stream, void* x, int act_dtype, int64_t n, int kind) {
-  PSAMD_REQUIRE(n >= 0 && kind >= 0 && kind <= 3, "bad size or activation");
+  PSAMD_REQUIRE(n >= 0 && kind >= 0 && kind <= 4, "bad size or activation");
   if (n == 0) return 0;
   PSAMD_REQUIRE(ceil_div(n, 256) <= 2147483647LL, "too large for one launch");
   hipStream_t s = static_cast<hipStream_t>(stream);

@@ -97,6 +97,8 @@ class StepContext:
     # Set by a block whose kernel adds a weighted sum of several outputs to the stream itself
     # (``parts.base.WeightedDeltas``); a sub-layer made of several then hands them over one by one.
     takes_weighted_deltas: bool = False
+    # The same for outputs that are normalized on their own first (``parts.base.NormedDeltas``).
+    takes_normed_deltas: bool = False
 
 
 class StepPacker:

@@ -19,7 +19,7 @@ from typing import Any, Sequence
 import torch
 
 from prefixserve_amd.build import ensure_kernels
-from prefixserve_amd.parts.base import NormedRows, ScaledDelta
+from prefixserve_amd.parts.base import NormedDeltas, NormedRows, ScaledDelta
 
 _F32, _BF16 = 0, 1
 _vp, _i32, _i64, _f32 = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_float
@@ -58,7 +58,7 @@ _SIGNATURES = {
     "psamd_linear_normed": [_vp, _vp, _vp, _vp, _i32, _f32, _vp, _vp, _i32, _i32, _i32, _i32, _i32],
     "psamd_qkv_rope_append_normed": [_vp, _vp, _vp, _i32, _f32, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _vp, _vp],
     "psamd_attention_generic": [_vp, _vp, _i32, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32,
-                                _vp, _vp, _i32],
+                                _vp, _vp, _i32, _vp, _i64],
     "psamd_attention_mfma_supports": [_i32, _i32, _i32],
     "psamd_attention_prefill_nsplit": [_i32, _i32, _i32, _i32, _i32],
     "psamd_attention_prefill_part_rows": [_i32, _i32, _i32],
@@ -70,9 +70,9 @@ _SIGNATURES = {
     "psamd_attention_decode": [_vp, _vp, _i32, _vp, _vp, _vp, _vp, _vp, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _i32,
                                _i32, _f32, _i32, _i32, _i32],
     "psamd_attention_prefill_extras": [_vp, _vp, _i32, _vp, _vp, _vp, _i32, _vp, _i32, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _i32,
-                                       _f32, _i32, _vp, _vp, _i32, _i32, _vp, _vp, _i32],
+                                       _f32, _i32, _vp, _vp, _i32, _i32, _vp, _vp, _i32, _vp, _i64],
     "psamd_attention_decode_extras": [_vp, _vp, _i32, _vp, _vp, _vp, _vp, _vp, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _i32,
-                                      _i32, _f32, _i32, _i32, _i32, _vp, _vp, _i32],
+                                      _i32, _f32, _i32, _i32, _i32, _vp, _vp, _i32, _vp, _i64],
     "psamd_sample": [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32],
     "psamd_scaled_add_rmsnorm": [_vp, _vp, _f32, _vp, _i32, _i32, _i64, _vp, _i32, _f32, _vp, _i32, _i64, _i32],
     "psamd_to_activation": [_vp, _vp, _vp, _i32, _i64],
@@ -88,13 +88,13 @@ _SIGNATURES = {
     "psamd_causal_conv": [_vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i64, _i32, _i32],
     "psamd_gated_scan": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _i32,
                          _vp, _i32, _i32, _vp, _i32, _vp, _i32, _i32, _i32],
-    "psamd_moe_route": [_vp, _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
-    "psamd_moe_topk": [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
+    "psamd_moe_route": [_vp, _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _vp, _i32, _i32, _i32, _f32, _i32, _vp],
+    "psamd_moe_topk": [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32, _i32, _i32, _f32, _i32, _vp],
     "psamd_moe_grouped_max_tiles": [_i64, _i32],
-    "psamd_moe_experts_grouped": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32, _i32,
+    "psamd_moe_experts_grouped": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32, _i32,
                                   _i32, _i32, _vp],
-    "psamd_moe_topk_group": [_vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _vp, _i32, _i32, _i32, _f32],
-    "psamd_moe_experts_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32,
+    "psamd_moe_topk_group": [_vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _vp, _i32, _i32, _i32, _f32, _i32, _vp],
+    "psamd_moe_experts_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32,
                                _i32, _i32, _vp],
     "psamd_row_gate": [_vp, _vp, _vp, _i32, _vp, _i64, _i32, _i32],
     "psamd_layernorm_step": [_vp, _vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _f32, _vp, _vp, _f32, _vp, _i32, _i64, _i32],
@@ -122,11 +122,19 @@ _SIGNATURES = {
                                     _f32, _i32, _i32, _vp, _vp, _vp, _i32, _vp, _i32],
     "psamd_attention_masked": [_vp, _vp, _i32, _vp, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32,
                                _vp, _vp, _vp, _i32, _vp],
+    "psamd_qkv_conv_append": [_vp, _vp, _i32, _i64, _vp, _i32, _i32, _i32, _i32, _vp, _vp, _i32, _f32, _vp, _vp, _vp, _vp, _vp,
+                              _vp, _i64, _vp, _vp, _vp, _i64, _i32],
+    "psamd_retention_powers": [],
+    "psamd_retention": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _vp, _vp, _i32, _vp, _f32, _vp, _i64, _vp, _vp, _vp, _i32,
+                        _i32, _vp, _i32, _vp, _i32, _vp, _i32, _i32, _i32, _i32, _f32, _vp],
+    "psamd_output_norm": [_vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _i32, _i32, _i64, _vp, _f32, _f32, _vp, _f32, _vp, _i32, _i64,
+                          _i32],
+    "psamd_embed_bigram": [_vp, _vp, _vp, _vp, _i32, _vp, _vp, _i64, _i32, _i32, _i64, _i64, _i64, _vp, _i64, _vp, _vp, _vp],
 }
 
 EXPERT_KINDS = {"gated": 0, "squared_relu": 1}
 
-ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3}
+ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3, "squared_relu": 4}
 
 
 GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
@@ -278,6 +286,22 @@ class HipOps:
         self._ok(self.lib.psamd_embed(self._stream(), ids.data_ptr(), table.data_ptr(), _code(table.dtype),
                                       out.data_ptr(), t, h, table.shape[0], float(factor)))
 
+    def embed_bigram(self, ids, table, bigram, out, copy, state, ctx, mul_prev: int, mul_cur: int) -> None:
+        """out (float32 [T, H]) = table[id] + bigram[(previous id * mul_prev + id * mul_cur) mod buckets], the last of bigram's
+        buckets + 1 rows for a sequence's first token; ``copy`` (or None): the same rows in the tables' dtype. ``state`` (int32
+        [slots, 1]): the item's last token + 1 (0: none), read and replaced."""
+        t, h = out.shape
+        self._need(ids.dtype == torch.int32 and ids.numel() == t == ctx.num_tokens, "embed_bigram: ids must be int32 [T]")
+        self._need(table.shape[1] == h and bigram.shape[1] == h and bigram.shape[0] >= 2 and table.dtype == bigram.dtype
+                   and table.is_contiguous() and bigram.is_contiguous(), "embed_bigram: tables of one dtype")
+        self._need(out.dtype == torch.float32 and out.is_contiguous(), "embed_bigram: bad output")
+        self._need(copy is None or (copy.shape == (t, h) and copy.dtype == table.dtype and copy.is_contiguous()), "embed_bigram: copy")
+        self._need(state.dtype == torch.int32 and state.dim() == 2 and state.is_contiguous(), "embed_bigram: state int32 [slots, 1]")
+        self._ok(self.lib.psamd_embed_bigram(self._stream(), ids.data_ptr(), table.data_ptr(), bigram.data_ptr(), _code(table.dtype),
+                                             out.data_ptr(), _ptr(copy), t, h, table.shape[0], bigram.shape[0] - 1, int(mul_prev),
+                                             int(mul_cur), state.data_ptr(), state.shape[1], ctx.tok_item.data_ptr(),
+                                             ctx.item_start.data_ptr(), ctx.slots.data_ptr()))
+
     def _delta_args(self, delta, t: int, h: int, out_dtype: torch.dtype) -> tuple:
         """(pointer, dtype code, slices, stride) of a delta: [T, H] in the activation dtype, or
         [S, T, H] float32 partial sums of a K-split product."""
@@ -333,6 +357,29 @@ class HipOps:
         self._ok(self.lib.psamd_scaled_add_rmsnorm(self._stream(), residual.data_ptr(), float(alpha), dptr, dcode, slices,
                                                    stride, weight.data_ptr(), _code(weight.dtype), float(eps), _ptr(out),
                                                    _code(out.dtype) if out is not None else _F32, t, h))
+
+    def output_norm(self, residual, delta, weight, eps: float, out) -> None:
+        """residual (float32 [T, H]) += weight * rmsnorm(delta); ``out`` (or None) receives the new rows in its dtype. ``delta``:
+        [T, H] in a kernel dtype, [S, T, H] float32 slices, or ``NormedDeltas`` of two of either."""
+        t, h = residual.shape
+        self._need(residual.dtype == torch.float32 and residual.is_contiguous(), "output_norm: the stream is float32")
+        self._need(weight.dtype == torch.float32 and weight.numel() == h and weight.is_contiguous(), "output_norm: weight")
+        if out is not None:
+            self._need(out.shape == (t, h) and out.is_contiguous(), "output_norm: bad output shape")
+        scale, in_eps = 1.0, 0.0
+        if isinstance(delta, NormedDeltas):
+            self._need(len(delta.parts) == 2, "output_norm: two outputs normalized on their own")
+            for _, w in delta.parts:
+                self._need(w.dtype == torch.float32 and w.numel() == h and w.is_contiguous(), "output_norm: the outputs' own weights")
+            (a, wa), (b, wb) = delta.parts
+            scale, in_eps = float(delta.scale), float(delta.eps)
+        else:
+            a, wa, b, wb = delta, None, None, None
+        ap, ac, an, ast = self._delta_args(a, t, h, a.dtype)
+        bp, bc, bn, bst = (None, _F32, 1, 0) if b is None else self._delta_args(b, t, h, b.dtype)
+        self._ok(self.lib.psamd_output_norm(self._stream(), residual.data_ptr(), ap, ac, an, ast, _ptr(wa), bp, bc, bn, bst, _ptr(wb), scale,
+                                            in_eps, weight.data_ptr(), float(eps), _ptr(out), _code(out.dtype) if out is not None else _F32,
+                                            t, h))
 
     def to_activation(self, src, out) -> None:
         """out = src (float32) in out's dtype."""
@@ -744,7 +791,7 @@ class HipOps:
     # ------------------------------------------------------------------ experts
 
     def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode: int = 0, groups: int = 0,
-                  keep: int = 0, factor: float = 1.0) -> None:
+                  keep: int = 0, factor: float = 1.0, group_max: bool = False, correction=None, identity: int = 0) -> None:
         """chosen[t, :], weight[t, :] = the experts with the largest sigmoid(x[t] . w_router[e]) and
         those scores, largest first, the lower index among equals; scores in 32-bit. With the router
         also given in the activation dtype (``w_router_act``), a step of more than
@@ -755,12 +802,20 @@ class HipOps:
         ``bias`` (float32 [E]) is added to the logits; ``mode`` 1: the largest logits are chosen and the
         weights are the softmax over the chosen logits alone. ``groups`` > 0: the experts form that many equal
         runs of neighbours, a run's score is the sum of its two largest scores, and only experts of the ``keep`` best
-        runs can be chosen. The weights are multiplied by ``factor``."""
+        runs can be chosen. The weights are multiplied by ``factor``. ``mode`` 2: the scores are the softmax over all logits,
+        the choice goes by score + ``correction`` (float32 [E]), the weights are the scores. ``group_max``: a run's score is
+        its largest alone. The last ``identity`` rows of the router are identity experts (``moe_experts``)."""
+        e, top = w_router.shape[0], chosen.shape[1]
+        if correction is not None:
+            self._need(correction.dtype == torch.float32 and correction.numel() == e and correction.is_contiguous(),
+                       "moe_route: the correction is float32 [E]")
+        self._need(0 <= identity < e, "moe_route: identity experts")
+        buckets = e - identity + (1 if identity else 0)       # what the pairs are sorted into: all identity pairs lie in one
+        rule = (_ptr(bias), int(mode), int(groups), int(keep), float(factor), int(group_max), _ptr(correction))
         if bias is not None:
             self._need(bias.dtype == torch.float32 and bias.numel() == w_router.shape[0] and bias.is_contiguous(),
                        "moe_route: the bias is float32 [E]")
         t, k = x.shape
-        e, top = w_router.shape[0], chosen.shape[1]
         if (w_router_act is not None and t > self.MOE_ROUTE_FUSED_MAX_TOKENS and w_router_act.dtype == x.dtype
                 and w_router_act.shape == w_router.shape and 1 <= top <= e):
             self._need(chosen.dtype == torch.int32 and weight.dtype == torch.float32 and chosen.shape == (t, top)
@@ -771,13 +826,12 @@ class HipOps:
             self._grouped_for = None
             if self._groups_pairs(x.dtype, t, k) and t <= self.MOE_CHOICE_SORTS_MAX_TOKENS and e <= 1024:
                 # A small step: the workgroup that chooses also sorts the pairs for the experts' kernels.
-                ints = self._group_ints(t, top, e)
+                ints = self._group_ints(t, top, buckets)
                 self._ok(self.lib.psamd_moe_topk_group(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
-                                                       ints.data_ptr(), t, e, top, _ptr(bias), int(mode), int(groups), int(keep), float(factor)))
-                self._grouped_for = (chosen.data_ptr(), t, top, e)
+                                                       ints.data_ptr(), t, e, buckets, top, *rule))
+                self._grouped_for = (chosen.data_ptr(), t, top, buckets)
                 return
-            self._ok(self.lib.psamd_moe_topk(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(), t, e, top,
-                                             _ptr(bias), int(mode), int(groups), int(keep), float(factor)))
+            self._ok(self.lib.psamd_moe_topk(self._stream(), logits.data_ptr(), chosen.data_ptr(), weight.data_ptr(), t, e, top, *rule))
             return
         self._grouped_for = None
         self._need(x.is_contiguous() and w_router.dtype == torch.float32 and w_router.is_contiguous()
@@ -786,8 +840,7 @@ class HipOps:
                    and weight.shape == (t, top) and chosen.is_contiguous() and weight.is_contiguous() and 1 <= top <= e,
                    "moe_route: outputs must be int32 and float32 [T, top]")
         self._ok(self.lib.psamd_moe_route(self._stream(), x.data_ptr(), _code(x.dtype), w_router.data_ptr(),
-                                          chosen.data_ptr(), weight.data_ptr(), t, k, e, top, _ptr(bias), int(mode), int(groups), int(keep),
-                                          float(factor)))
+                                          chosen.data_ptr(), weight.data_ptr(), t, k, e, top, *rule))
 
     def _groups_pairs(self, dtype: torch.dtype, t: int, k: int) -> bool:
         """Whether a step of ``t`` tokens of width ``k`` runs its experts grouped by expert."""
@@ -798,13 +851,15 @@ class HipOps:
         return self.ws.get("moe.group", (t * top + 3 * tiles,), torch.int32)
 
     def moe_experts(self, x, chosen, weight, w_in, w_down, act, out, gate_alpha: float, limit: float,
-                    up_shift: float, weight_on_output: bool = False, kind: str = "gated", residual=None, col_scale=None) -> None:
+                    up_shift: float, weight_on_output: bool = False, kind: str = "gated", residual=None, col_scale=None,
+                    identity: int = 0) -> None:
         """out[j, t] = down_e(act_e(weight[t, j] * x[t])) for e = chosen[t, j], as float32 slices [top, T, K];
         ``act`` [T * top, F] is scratch in the activation dtype. ``weight_on_output``: out[j, t] =
         weight[t, j] * down_e(act_e(x[t])) instead. ``kind`` "gated": ``w_in`` is [E, 2F, K], gate rows in front of up
         rows; "squared_relu": [E, F, K], act_e(h) = max(w_in h, 0)^2. ``residual`` (float32 [T, K], instead of
         ``out``, which is then None; bfloat16 only): every pair adds its output, times ``col_scale`` (float32 [K]) if
-        given, into it with float atomics."""
+        given, into it with float atomics. Choices from E on (``identity`` of them) are identity experts, whose output is
+        weight[t, j] * x[t]."""
         t, k = x.shape
         top = chosen.shape[1]
         e, _, f = w_down.shape
@@ -830,17 +885,18 @@ class HipOps:
         tail = (int(weight_on_output), EXPERT_KINDS[kind], int(into), _ptr(col_scale))
         if self._groups_pairs(x.dtype, t, k) and f % 8 == 0:
             # Sorted by expert and run in tiles on the matrix cores: an expert is read once per tile of pairs.
-            ints = self._group_ints(t, top, e)
-            done = int(getattr(self, "_grouped_for", None) == (chosen.data_ptr(), t, top, e))   # the router's kernel sorted them
+            buckets = e + (1 if identity else 0)
+            ints = self._group_ints(t, top, buckets)
+            done = int(getattr(self, "_grouped_for", None) == (chosen.data_ptr(), t, top, buckets))   # the router's kernel sorted them
             self._grouped_for = None
             self._ok(self.lib.psamd_moe_experts_grouped(self._stream(), x.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
                                                         w_in.data_ptr(), w_down.data_ptr(), act.data_ptr(),
-                                                        out.data_ptr(), ints.data_ptr(), t, k, f, e, top, float(gate_alpha),
+                                                        out.data_ptr(), ints.data_ptr(), t, k, f, e, int(identity), top, float(gate_alpha),
                                                         float(limit), float(up_shift), done, *tail))
             return
         self._ok(self.lib.psamd_moe_experts_rows(self._stream(), x.data_ptr(), chosen.data_ptr(), weight.data_ptr(),
                                                  w_in.data_ptr(), w_down.data_ptr(), act.data_ptr(), out.data_ptr(),
-                                                 _code(x.dtype), t, k, f, e, top, float(gate_alpha), float(limit),
+                                                 _code(x.dtype), t, k, f, e, int(identity), top, float(gate_alpha), float(limit),
                                                  float(up_shift), *tail))
 
     def row_gate(self, out, x, w) -> None:
@@ -910,6 +966,77 @@ class HipOps:
                                               ctx.item_start.data_ptr(), ctx.slots.data_ptr(), t, ctx.num_items, channels, taps,
                                               int(silu)))
 
+    def qkv_conv_append(self, rows, col: int, conv_w, hq: int, hkv: int, d: int, positions, table, norm_dim: int, norm_eps: float,
+                        q_weight, k_weight, q_out, kv, write_slot, state, state_offset: int, ctx) -> None:
+        """From a product's rows (hq q heads, hkv k heads, hkv v heads of d channels from column ``col`` on) to what attention reads:
+        every channel through a causal convolution (``conv_w`` float32 [taps, channels], the last tap the token's own; in front of an
+        item's first token come the inputs saved in ``state[slot, state_offset + j * channels + c]``, which are then replaced), q
+        and k heads divided by their root mean square over ``norm_dim`` (0: not), times ``q_weight`` / ``k_weight`` (float32 [d] or None),
+        rotated (pairs (i, i + d/2); ``table`` or None); q to ``q_out`` [T, hq * d], k and v to their pages (``kv`` None: nowhere)."""
+        t = q_out.shape[0]
+        taps, channels = conv_w.shape
+        self._need(channels == (hq + 2 * hkv) * d and conv_w.dtype == torch.float32 and conv_w.is_contiguous(), "qkv_conv_append: taps [taps, channels]")
+        self._need(rows.dim() == 2 and rows.is_contiguous() and rows.shape[0] == t == ctx.num_tokens and 0 <= col
+                   and col + channels <= rows.shape[1], "qkv_conv_append: rows")
+        self._need(q_out.shape == (t, hq * d) and q_out.dtype == rows.dtype and q_out.is_contiguous(), "qkv_conv_append: queries")
+        self._need(positions.dtype == torch.int32 and positions.numel() == t, "qkv_conv_append: positions")
+        for v in (q_weight, k_weight):
+            self._need(v is None or (v.dtype == torch.float32 and v.numel() == d and v.is_contiguous()), "qkv_conv_append: norm weights")
+        if table is not None:
+            self._need(table.dtype == torch.float32 and table.shape[1:] == (d // 2, 2) and table.is_contiguous() and table.shape[0] >= 1,
+                       "qkv_conv_append: table must be float32 [positions, D/2, 2]")
+        if kv is not None:
+            self._need(kv.dtype == rows.dtype and kv.shape[1:] == (2, hkv, 16 * d) and kv.is_contiguous(),
+                       "qkv_conv_append: cache must be [blocks, 2, kv_heads, 16*D] in the activation dtype")
+            self._need(write_slot.dtype == torch.int32 and write_slot.numel() == t, "qkv_conv_append: write slots")
+        sptr, srow = None, 0
+        if taps > 1:
+            self._need(state is not None and state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous() and 0 <= state_offset
+                       and state_offset + (taps - 1) * channels <= state.shape[1], "qkv_conv_append: the state's saved inputs")
+            sptr, srow = state.data_ptr() + 4 * state_offset, state.shape[1]
+        self._ok(self.lib.psamd_qkv_conv_append(
+            self._stream(), rows.data_ptr() + col * rows.element_size(), _code(rows.dtype), rows.shape[1], conv_w.data_ptr(), taps, hq, hkv, d,
+            positions.data_ptr(), _ptr(table), int(norm_dim), float(norm_eps), _ptr(q_weight), _ptr(k_weight), q_out.data_ptr(), _ptr(kv),
+            None if kv is None else write_slot.data_ptr(), sptr, srow, ctx.tok_item.data_ptr(), ctx.item_start.data_ptr(),
+            ctx.slots.data_ptr(), t, ctx.num_items))
+
+    # ------------------------------------------------------------ retention
+
+    def retention_powers(self) -> int:
+        """How many powers of a head's decay ``retention`` wants, from the zeroth on."""
+        return int(self.lib.psamd_retention_powers())
+
+    def retention(self, rows, q_col: int, k_col: int, v_col: int, g_col: int, table, powers, k_scale: float, state, state_offset: int, ctx,
+                  heads: int, dim_p: int, vdim_p: int, vdim: int, eps: float, out) -> None:
+        """Linear attention with a fixed decay per head over each item's tokens from its state slot: q, k rotated (``table`` float32
+        [pos, rot/2, 2], pairs (i, i + rot/2) of the first rot dimensions; None: not), k times ``k_scale``, S <- decay S + k v^T, o = S^T q,
+        out = o / sqrt(mean(o^2) + eps) * silu(gate), per head, the mean over ``vdim``. ``rows`` hold q and k (heads of ``dim_p``), v and gate
+        (heads of ``vdim_p``) from their columns on, sizes padded with zeros to multiples of 16. ``powers`` float32 [heads,
+        ``retention_powers()``]. The state of a head is float32 [dim_p, vdim_p], heads one behind the other from ``state_offset`` on."""
+        t = out.shape[0]
+        self._need(rows.dim() == 2 and rows.is_contiguous() and rows.shape[0] == t == ctx.num_tokens, "retention: rows")
+        self._need(out.dtype == rows.dtype and out.shape == (t, heads * vdim_p) and out.is_contiguous(), "retention: out")
+        self._need(powers.dtype == torch.float32 and powers.shape == (heads, self.retention_powers()) and powers.is_contiguous(), "retention: powers")
+        rot = 0
+        if table is not None:
+            self._need(table.dtype == torch.float32 and table.dim() == 3 and table.shape[2] == 2 and table.is_contiguous(), "retention: table")
+            rot = 2 * table.shape[1]
+        self._need(state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous() and 0 <= state_offset
+                   and state_offset + heads * dim_p * vdim_p <= state.shape[1], "retention: the state")
+        n_blocks = int(ctx.num_prefill_blocks)
+        sums = None
+        if n_blocks:
+            # Room for the most runs of a step of this many tokens (every request's last run may be short), so that a
+            # smaller step of more requests does not grow the buffer.
+            most = t // 128 + state.shape[0]
+            self._need(n_blocks <= most, "retention: more runs than tokens and slots allow")
+            sums = self.ws.get("retention.sums", (most * heads * dim_p * vdim_p,), torch.float32)
+        self._ok(self.lib.psamd_retention(
+            self._stream(), rows.data_ptr(), _code(rows.dtype), rows.shape[1], q_col, k_col, v_col, g_col, ctx.positions.data_ptr(), _ptr(table), rot,
+            powers.data_ptr(), float(k_scale), state.data_ptr() + 4 * state_offset, state.shape[1], ctx.item_start.data_ptr(),
+            ctx.slots.data_ptr(), ctx.pf_tiles.data_ptr(), ctx.num_prefill_tiles, self.PREFILL_TILE_Q, ctx.pf_blocks.data_ptr(), n_blocks,
+            ctx.dec_items.data_ptr(), ctx.num_decode, _ptr(sums), heads, dim_p, vdim_p, vdim, float(eps), out.data_ptr()))
+
     # ------------------------------------------ several streams, mixers side by side, recurrences through the delta scan
 
     def stream_rms_norm(self, x, weight, eps: float) -> None:
@@ -954,7 +1081,7 @@ class HipOps:
                                              float(b_scale), out.data_ptr(), t * h))
 
     def activation(self, x, kind: str) -> None:
-        """x <- f(x) in place: "gelu" (exact), "gelu_tanh", "silu" or "relu"."""
+        """x <- f(x) in place: "gelu" (exact), "gelu_tanh", "silu", "relu" or "squared_relu"."""
         self._need(x.is_contiguous(), "activation: a contiguous tensor")
         self._ok(self.lib.psamd_activation(self._stream(), x.data_ptr(), _code(x.dtype), x.numel(), ACTIVATIONS[kind]))
 
@@ -1165,14 +1292,23 @@ class HipOps:
 
     def paged_attention(self, qkv, out, kv, ctx, group: int, hq: int, hkv: int, d: int, scale: float,
                         window: int | None, exact_weights: bool = False, sink=None, dist_bias=None, keep_first: int = 0,
-                        pooled=None, head_gate=None) -> None:
+                        pooled=None, head_gate=None, out_gate=None) -> None:
         """``exact_weights``: the softmax weights enter the product with the values as computed in
         32-bit (the matrix-core kernels then take them as three bfloat16 terms that sum to the float32
         weight exactly) instead of rounded to bfloat16; the 32-bit kernels always do. ``sink``
         (float32 [hq]): exp(sink) joins every softmax's denominator. ``dist_bias`` (float32 [hq, n]):
         entry [h, min(i - j, n - 1)] is added to the scaled score of query i and key j. ``keep_first``: the window also
         sees the first that many positions. ``pooled`` = (pages, group, block): one mean key and value per block of tokens
-        wholly in front of the window, from pages of their own. ``head_gate`` (float32 [T, hq]): output times sigmoid."""
+        wholly in front of the window, from pages of their own. ``head_gate`` (float32 [T, hq]): output times sigmoid.
+        ``out_gate`` = (rows, column): output entry (t, h d + i) times sigmoid(rows[t, column + h d + i]), rows in the
+        activation dtype."""
+        gate = (None, 0)
+        if out_gate is not None:
+            rows, col = out_gate
+            self._need(keep_first == 0 and pooled is None and head_gate is None, "attention: one kind of gate")
+            self._need(rows.dtype == qkv.dtype and rows.dim() == 2 and rows.is_contiguous() and rows.shape[0] == qkv.shape[0]
+                       and col >= 0 and col + hq * d <= rows.shape[1] and rows.shape[1] % 4 == 0 and col % 4 == 0, "attention: the gate's columns")
+            gate = (rows.data_ptr() + col * rows.element_size(), rows.shape[1])
         if keep_first or pooled is not None or head_gate is not None:
             self._need(sink is None and dist_bias is None and window is not None and window >= 1,
                        "attention: kept positions, pooled blocks and a gate per head go with a window and without sink or bias")
@@ -1212,7 +1348,7 @@ class HipOps:
         if dist_bias is not None:
             self._need(dist_bias.dtype == torch.float32 and dist_bias.dim() == 2 and dist_bias.shape[0] == hq
                        and dist_bias.shape[1] >= 1 and dist_bias.is_contiguous(), "attention: distance bias is float32 [hq, n]")
-        extras = sink is not None or dist_bias is not None
+        extras = sink is not None or dist_bias is not None or out_gate is not None
         t = qkv.shape[0]
         g = ctx.groups[group]
         self._need(out.shape == (t, hq * d) and out.is_contiguous() and out.dtype == qkv.dtype, "attention: output")
@@ -1238,7 +1374,7 @@ class HipOps:
                 part_ml = self.ws.get("attn.prefill_part_ml", (rows * hq * 2,), torch.float32)
                 if nsplit > 1:
                     self._need(32 * ctx.num_prefill_tiles * nsplit <= rows, "attention: more split tiles than planned for")
-                tail = (_ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1]) if extras else ()
+                tail = (_ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1], *gate) if extras else ()
                 self._ok((self.lib.psamd_attention_prefill_extras if extras else self.lib.psamd_attention_prefill)(
                     s, qkv.data_ptr(), stride, out.data_ptr(), kv.data_ptr(), ctx.pf_tiles.data_ptr(),
                     ctx.num_prefill_tiles, ctx.pf_blocks.data_ptr(), ctx.num_prefill_blocks, kv_len,
@@ -1257,7 +1393,7 @@ class HipOps:
                 self._need(ctx.num_decode * nsplit <= parts, "attention: more (request, run) pairs than planned for")
                 part_o = self.ws.get("attn.part_o", (parts * hq * d,), torch.float32)
                 part_ml = self.ws.get("attn.part_ml", (parts * hq * 2,), torch.float32)
-                tail = (_ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1]) if extras else ()
+                tail = (_ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1], *gate) if extras else ()
                 self._ok((self.lib.psamd_attention_decode_extras if extras else self.lib.psamd_attention_decode)(
                     s, qkv.data_ptr(), stride, out.data_ptr(), kv.data_ptr(), part_o.data_ptr(), part_ml.data_ptr(),
                     ctx.dec_items.data_ptr(), ctx.num_decode, ctx.item_start.data_ptr(),
@@ -1267,7 +1403,7 @@ class HipOps:
         self._ok(self.lib.psamd_attention_generic(
             s, qkv.data_ptr(), stride, out.data_ptr(), kv.data_ptr(), _code(qkv.dtype), t, ctx.positions.data_ptr(),
             ctx.tok_item.data_ptr(), g.table_off.data_ptr(), g.block_ids.data_ptr(), hq, hkv, d, scale, win,
-            _ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1]))
+            _ptr(sink), _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1], *gate))
 
     # ---------------------------------------------------------------- sampling
 

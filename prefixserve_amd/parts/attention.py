@@ -8,7 +8,7 @@ from typing import TYPE_CHECKING, Any, Mapping
 
 import torch
 
-from .base import CacheNeed, Mixer, PositionEncoding, RotaryTable, Runtime, WeightWant, register_mixer
+from .base import CacheNeed, Mixer, PositionEncoding, RotaryTable, Runtime, StateNeed, WeightWant, register_mixer
 
 if TYPE_CHECKING:
     from prefixserve_amd.engine.batch import StepContext
@@ -42,13 +42,16 @@ def slot_size(head_dim: int, value_dim: int, largest: int = 256) -> int:
     raise ValueError(f"head sizes up to {largest} are implemented, got {need}")
 
 
-def head_slots(head_dim: int, rotary_dim: int, slots: int) -> list[int]:
+def head_slots(head_dim: int, rotary_dim: int, slots: int, neighbours: bool = False) -> list[int]:
     """Slot of each of a head's ``head_dim`` dimensions in a head of ``slots`` slots whose pair
-    (i, i + slots/2) rotates together. The model's partners (i, i + rotary_dim/2), i < rotary_dim/2,
-    go to (i, i + slots/2); the dimensions that do not rotate fill the first half's remaining
-    slots and then the second half's (their table entries are the identity)."""
+    (i, i + slots/2) rotates together. The model's partners (i, i + rotary_dim/2), or (2i, 2i + 1) for
+    ``neighbours``, i < rotary_dim/2, go to (i, i + slots/2); the dimensions that do not rotate fill the
+    first half's remaining slots and then the second half's (their table entries are the identity)."""
     half, r2 = slots // 2, rotary_dim // 2
-    out = [i if i < r2 else half + (i - r2) for i in range(rotary_dim)]
+    if neighbours:
+        out = [i // 2 if i % 2 == 0 else half + i // 2 for i in range(rotary_dim)]
+    else:
+        out = [i if i < r2 else half + (i - r2) for i in range(rotary_dim)]
     free = list(range(r2, half)) + list(range(half + r2, slots))
     out += free[: head_dim - rotary_dim]
     assert len(out) == head_dim and len(set(out)) == head_dim
@@ -118,8 +121,20 @@ class PagedAttention(Mixer):
       cache entry of their own with one place per P tokens (``aux_cache_needs``: "pool"), written
       when the block's last token runs; tokens that have left the window and whose block is not
       complete in front of it are not seen.
+    * ``pairs`` "neighbours": the rotation's partners are (2i, 2i + 1) instead of (i, i + rotary_dim/2); they are laid
+      apart at bind time.
+    * ``conv_taps`` = n: every channel of q, k and v passes a causal convolution over n tokens (names "q_conv", "k_conv",
+      "v_conv", [channels, n], the last tap the token's own, zeros in front of the sequence) behind the projection. The last
+      n - 1 projected rows are the mixer's state.
+    * ``norm_first``: the q/k norm (with ``qk_norm_weights``) comes in front of the rotation instead of behind it.
+    * ``out_gate``: the heads' outputs are multiplied entry by entry by sigmoid(W_g x) (name "gate", [heads * value_dim,
+      hidden]) in front of the output matrix.
+      These three run through one product [q | k | v | gate] and one kernel for convolution, norm, rotation and cache write
+      (``ops.qkv_conv_append``); a container may form that product for them (``takes_input_rows``).
     * ``head_gate``: a number per query head and token, sigmoid(W x)_h (name "head_gate",
       [heads, hidden]), multiplies the head's output before the output matrix; 32-bit."""
+
+    state_in_graphs = True
 
     def __init__(self, hidden_size: int, positions: Mapping[str, PositionEncoding], num_heads: int,
                  num_kv_heads: int, head_dim: int, names: Mapping[str, str], position: str | None = None,
@@ -127,7 +142,8 @@ class PagedAttention(Mixer):
                  qk_norm_eps: float | None = None, own_kv: bool = True, exact_weights: bool = False,
                  qk_bias: bool = False, qk_norm_weights: bool = False, values_are_keys: bool = False,
                  sink: bool = False, distance_bias: Mapping[str, Any] | None = None, head_scale: bool = False,
-                 keep_first: int = 0, pooled_block: int = 0, head_gate: bool = False) -> None:
+                 keep_first: int = 0, pooled_block: int = 0, head_gate: bool = False, pairs: str = "halves",
+                 conv_taps: int = 0, norm_first: bool = False, out_gate: bool = False) -> None:
         if num_kv_heads < 1 or num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads not divisible by {num_kv_heads} kv heads")
         self.hidden_size = int(hidden_size)
@@ -159,6 +175,15 @@ class PagedAttention(Mixer):
         self.masked = bool(self.keep_first or self.pooled_block or self.head_gate)
         if self.masked and (self.has_sink or self.distance_bias is not None):
             raise ValueError("kept positions, pooled blocks and a gate per head are not combined with a sink or a distance bias")
+        if pairs not in ("halves", "neighbours") or not 0 <= int(conv_taps) <= 16:
+            raise ValueError(f"pairs {pairs!r}, {conv_taps} taps (at most 16)")
+        self.conv_taps, self.out_gate, self.norm_first = int(conv_taps), bool(out_gate), bool(norm_first)
+        self.neighbours = pairs == "neighbours"
+        self.takes_input_rows = bool(self.conv_taps or self.out_gate or self.norm_first)
+        if self.takes_input_rows and (self.masked or self.qk_bias or self.values_are_keys or self.head_scale or not self.own_kv
+                                      or (self.qk_norm_eps is not None and not self.norm_first)):
+            raise ValueError("convolutions, a gate on the output and a norm in front of the rotation go with keys and values of the "
+                             "layer's own, and without biases, factors per head, kept positions, blocks or a norm behind the rotation")
         self.bias = self.q_norm_weight = self.k_norm_weight = self.sink = self.distance_table = None
         self.names = dict(names)
         self.window = None if window is None else int(window)
@@ -168,7 +193,7 @@ class PagedAttention(Mixer):
             raise ValueError("PagedAttention applies rotation tables; other encodings belong to their own mixer")
         rotary = self.head_dim if self.pos is None or self.pos.rotary_dim is None else int(self.pos.rotary_dim)
         self.plain = (self.value_dim == self.head_dim and rotary == self.head_dim and self.qk_norm_eps is None
-                      and self.own_kv and not extras)
+                      and self.own_kv and not extras and not self.takes_input_rows and not self.neighbours)
         if self.plain:
             if head_dim % 16 or not 16 <= head_dim <= 256:
                 raise ValueError(f"head_dim must be a multiple of 16 in [16, 256], got {head_dim}")
@@ -178,13 +203,14 @@ class PagedAttention(Mixer):
             if self.head_dim < 1 or self.value_dim < 1 or rotary > self.head_dim:
                 raise ValueError(f"bad head sizes: {self.head_dim}, {self.value_dim}, rotating {rotary}")
             self.slots = slot_size(self.head_dim, self.value_dim)
-            self.index = head_slots(self.head_dim, rotary, self.slots)
+            self.index = head_slots(self.head_dim, rotary, self.slots, self.neighbours)
         if isinstance(self.pos, RotaryTable) and self.pos.head_dim != self.slots:
             raise ValueError(f"the rotation table is made for heads of {self.pos.head_dim}, attention runs with {self.slots}")
         # The norm kernels in front may be skipped only by the form whose first kernel normalizes.
         self.takes_normed_rows = self.plain
         self.q_size = self.num_heads * self.slots
         self.kv_size = self.num_kv_heads * self.slots if self.own_kv else 0
+        self.channels = self.q_size + 2 * self.kv_size               # what a convolution runs over: [q | k | v]
         self.row_width = self.q_size + (1 if self.values_are_keys else 2) * self.kv_size
 
     def weights(self) -> dict[str, WeightWant]:
@@ -210,7 +236,28 @@ class PagedAttention(Mixer):
             want[n["rel"]] = WeightWant((self.distance_bias[0], self.num_heads), "bias")
         if self.head_gate:
             want[n["head_gate"]] = WeightWant((self.num_heads, h))
+        if self.conv_taps:
+            for which, size in (("q_conv", self.num_heads * self.head_dim), ("k_conv", self.num_kv_heads * self.head_dim),
+                                ("v_conv", self.num_kv_heads * self.value_dim)):
+                want[n[which]] = WeightWant((size, self.conv_taps), "bias")
+        if self.out_gate:
+            want[n["gate"]] = WeightWant((self.num_heads * self.value_dim, h))
         return want
+
+    def state_need(self) -> StateNeed | None:
+        return StateNeed(((self.conv_taps - 1) * self.channels,), torch.float32) if self.conv_taps > 1 else None
+
+    def input_matrix(self, tensors: Mapping[str, torch.Tensor]) -> torch.Tensor:
+        """Rows of q, k, v (and the gate), heads laid into their slots."""
+        n = self.names
+        rows = [self._spread(tensors[n["q"]], self.num_heads, self.head_dim, self.index)]
+        if self.own_kv:
+            rows.append(self._spread(tensors[n["k"]], self.num_kv_heads, self.head_dim, self.index))
+            if not self.values_are_keys:
+                rows.append(self._spread(tensors[n["v"]], self.num_kv_heads, self.value_dim, None))
+        if self.out_gate:
+            rows.append(self._spread(tensors[n["gate"]], self.num_heads, self.value_dim, None))
+        return torch.cat(rows, dim=0)
 
     def cache_need(self) -> CacheNeed:
         if self.pooled_block:
@@ -239,12 +286,7 @@ class PagedAttention(Mixer):
             self.w_qkv = rt.ops.prepare_matrix(torch.cat([tensors[n["q"]], tensors[n["k"]], tensors[n["v"]]], dim=0), rt)
             self.w_o = rt.ops.prepare_matrix(tensors[n["o"]], rt)
             return
-        rows = [self._spread(tensors[n["q"]], self.num_heads, self.head_dim, self.index)]
-        if self.own_kv:
-            rows.append(self._spread(tensors[n["k"]], self.num_kv_heads, self.head_dim, self.index))
-            if not self.values_are_keys:
-                rows.append(self._spread(tensors[n["v"]], self.num_kv_heads, self.value_dim, None))
-        self.w_qkv = rt.ops.prepare_matrix(torch.cat(rows, dim=0), rt)
+        self.w_qkv = None if self.input_elsewhere else rt.ops.prepare_matrix(self.input_matrix(tensors), rt)
         o = tensors[n["o"]]
         wide = torch.zeros((o.shape[0], self.num_heads, self.slots), dtype=o.dtype)
         # A value that is the key lies in the key's slots.
@@ -260,6 +302,15 @@ class PagedAttention(Mixer):
             both = [self._spread(tensors[n[key]].to(torch.float32)[:, None], heads, self.head_dim, self.index)
                     for key, heads in (("q_bias", self.num_heads), ("k_bias", self.num_kv_heads))]
             self.bias = on_device(torch.cat(both, dim=0).view(-1))
+        if self.takes_input_rows:
+            # [taps, channels], a convolution's channels laid out like the product's; without one, a single tap of one.
+            if self.conv_taps:
+                taps = [self._spread(tensors[n[which]].to(torch.float32), heads, size, index) for which, heads, size, index in (
+                    ("q_conv", self.num_heads, self.head_dim, self.index), ("k_conv", self.num_kv_heads, self.head_dim, self.index),
+                    ("v_conv", self.num_kv_heads, self.value_dim, None))]
+                self.conv_w = on_device(torch.cat(taps, dim=0).t())
+            else:
+                self.conv_w = on_device(torch.ones((1, self.channels)))
         self.q_weight_per_head = False
         if self.qk_norm_weights:
             self.q_norm_weight = on_device(self._spread(tensors[n["q_norm"]].to(torch.float32)[:, None], 1, self.head_dim, self.index).view(-1))
@@ -281,7 +332,7 @@ class PagedAttention(Mixer):
 
     def weight_bytes(self) -> int:
         gate = self.w_gate.numel() * self.w_gate.element_size() if self.head_gate else 0
-        return sum(w.numel() * w.element_size() for w in (self.w_qkv, self.w_o)) + gate
+        return sum(w.numel() * w.element_size() for w in (self.w_qkv, self.w_o) if w is not None) + gate
 
     def forward(self, x: torch.Tensor, ctx: "StepContext", cache: Any, state: torch.Tensor | None,
                 writes_cache: bool) -> torch.Tensor:
@@ -290,6 +341,10 @@ class PagedAttention(Mixer):
         table = self.pos.table if self.pos is not None else None
         if writes_cache and not self.own_kv:
             raise ValueError("a layer without keys and values of its own cannot write a cache entry")
+        if self.takes_input_rows:
+            rows = ws.get("attn.in", (t, self.w_qkv.shape[0]), rt.dtype)
+            ops.linear(x, self.w_qkv, rows)
+            return self.forward_rows(rows, 0, ctx, cache, state, writes_cache)
         if self.plain:
             qkv = ws.get("attn.qkv", (t, self.q_size + 2 * self.kv_size), rt.dtype)
             ops.qkv_rope_append(x, self.w_qkv, qkv, self.num_heads, self.num_kv_heads, self.head_dim, ctx.positions, table,
@@ -342,6 +397,23 @@ class PagedAttention(Mixer):
         else:
             ops.paged_attention(qkv, out, cache.kv, ctx, cache.group, self.num_heads, self.num_kv_heads,
                                 self.slots, self.scale, cache.window)
+        return ops.linear_to_residual(out, self.w_o, "attn.delta", getattr(ctx, "residual", None))
+
+
+    def forward_rows(self, rows: torch.Tensor, col: int, ctx: "StepContext", cache: Any, state: torch.Tensor | None,
+                     writes_cache: bool) -> torch.Tensor | None:
+        """From the product's rows, [q | k | v | gate] from column ``col`` on."""
+        rt, ops, ws = self.rt, self.rt.ops, self.rt.workspace
+        t = rows.shape[0]
+        norm_dim, eps = (self.head_dim, self.qk_norm_eps) if self.qk_norm_eps is not None else (0, 0.0)
+        q = ws.get("attn.q", (t, self.q_size), rt.dtype)
+        ops.qkv_conv_append(rows, col, self.conv_w, self.num_heads, self.num_kv_heads, self.slots, ctx.positions,
+                            self.pos.table if self.pos is not None else None, norm_dim, eps, self.q_norm_weight, self.k_norm_weight, q,
+                            cache.kv if writes_cache else None, ctx.groups[cache.group].write_slot, state, self.state_base, ctx)
+        out = ws.get("attn.out", (t, self.q_size), rt.dtype)
+        ops.paged_attention(q, out, cache.kv, ctx, cache.group, self.num_heads, self.num_kv_heads, self.slots, self.scale, cache.window,
+                            exact_weights=self.exact_weights, sink=self.sink, dist_bias=self.distance_table,
+                            out_gate=(rows, col + self.channels) if self.out_gate else None)
         return ops.linear_to_residual(out, self.w_o, "attn.delta", getattr(ctx, "residual", None))
 
 

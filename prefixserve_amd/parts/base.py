@@ -140,6 +140,18 @@ class WeightedDeltas:
 
 
 @dataclass
+class NormedDeltas:
+    """What a sub-layer made of several hands on when each output is normalized on its own: scale times the sum over
+    ``parts`` of weight * d / sqrt(mean(d^2) + eps), (d, weight) each, weights float32 [hidden] and d in one of the forms
+    ``Mixer.forward`` may return. Formed in 32-bit by the kernel that adds it to the stream (``ops.output_norm``), for a
+    block that says it takes such (``ctx.takes_normed_deltas``)."""
+
+    parts: "list[tuple[torch.Tensor, torch.Tensor]]"
+    scale: float
+    eps: float
+
+
+@dataclass
 class Runtime:
     """What every part needs to run: the device, the activation dtype (bfloat16 for
     serving, float32 for the exact path), the kernel bindings and the buffer store."""
@@ -194,6 +206,13 @@ class Norm(Part):
         raise NotImplementedError
 
 
+    def add_output(self, residual: torch.Tensor, delta: "torch.Tensor | NormedDeltas", out_name: str) -> torch.Tensor:
+        """The norm on the output alone: residual (float32 [T,H], in place) += norm(delta), all of it in
+        32-bit; ``delta`` as for ``add_norm`` (never None), or ``NormedDeltas``. Returns the new stream in the
+        activation dtype (the stream itself when that is float32)."""
+        raise NotImplementedError
+
+
 class PositionEncoding(Part):
     """Position information applied to queries and keys before attention."""
 
@@ -239,6 +258,13 @@ class Mixer(Part):
     # parts' states side by side and sets this before the first step.
     state_base = 0
 
+    # True: the mixer reads x through one input matrix alone and can be handed the product: ``input_matrix(tensors)`` gives
+    # the matrix [n, hidden] (on the host) and ``forward_rows(rows, col, ctx, cache, state, writes_cache)`` runs from
+    # ``rows`` [T, >= col + n] in the activation dtype. A container of several such mixers forms one product for all.
+    takes_input_rows = False
+    # ... set by such a container before ``bind``: the mixer then keeps no copy of that matrix itself.
+    input_elsewhere = False
+
     # True: ``forward`` takes ``NormedRows`` for x (it hands x to kernels that normalize their
     # tokens themselves); the block then lets the norm in front of it be lazy.
     takes_normed_rows = False
@@ -271,6 +297,18 @@ class Transform(Part):
     behind the token table, or the logits ``[S, vocab]``. ``rows`` are the flat token rows the
     tensor's rows belong to (all tokens in order for the stream, ``ctx.logit_rows`` for logits),
     for a transform that depends on the position (``ctx.positions[rows]``)."""
+
+    # The first transform behind the token table may do the gather itself: ``gather(ids, table, out, ctx, state, copy)``
+    # writes the transformed rows to ``out`` (float32 [T, hidden]) and, where ``copy`` is given, the same rows in the
+    # activation dtype.
+    gather = None
+
+    # Per-request state of fixed size, as for ``Mixer`` (whose rules about clearing and captured steps hold here too):
+    # for transforms behind the token table, which get it as ``state`` in ``gather``.
+    state_in_graphs = False
+
+    def state_need(self) -> StateNeed | None:
+        return None
 
     # A transform of the stream may offer ``add_pending(t, pending, ctx)``: what the last sub-layer left
     # to be added and then the transform itself, in one go.

@@ -211,7 +211,51 @@ class SandwichBlock:
         return None
 
 
+class OutputNormBlock:
+    """A norm on each sub-layer's output and none elsewhere: x <- x + norm1(mixer(x)), then, when the layer has a
+    feed-forward, x <- x + norm2(feed_forward(x)). The sub-layers read the stream itself, in the activation dtype.
+
+    The sub-layers hand their output back (``ctx.residual`` is None while they run); one kernel per sub-layer sums it up,
+    normalizes it, adds it into the float32 stream and writes the stream's copy that the next sub-layer reads
+    (``ctx.stream_copy``). A mixer made of two whose outputs are normalized on their own first leaves that to the same
+    kernel (``ctx.takes_normed_deltas``). Nothing is left pending."""
+
+    reads_stream_copy = True
+
+    def __init__(self, mixer: Mixer, feed_forward: FeedForward | None, mixer_norm: Norm, feed_forward_norm: Norm | None) -> None:
+        if (feed_forward is None) != (feed_forward_norm is None):
+            raise ValueError("a feed-forward comes with its norm, a layer without one has none")
+        self.mixer, self.feed_forward = mixer, feed_forward
+        self.mixer_norm, self.feed_forward_norm = mixer_norm, feed_forward_norm
+
+    def parts(self) -> list[Part]:
+        return [p for p in (self.mixer, self.mixer_norm, self.feed_forward, self.feed_forward_norm) if p is not None]
+
+    def forward(self, residual: torch.Tensor, pending: torch.Tensor | None, ctx: "StepContext", cache: Any,
+                state: torch.Tensor | None, writes_cache: bool) -> None:
+        rt = self.mixer_norm.rt
+        if pending is not None:
+            rt.ops.residual_add(residual, pending)
+            ctx.stream_copy = None
+        x = residual if rt.dtype == torch.float32 else ctx.stream_copy
+        if x is None:
+            x = rt.workspace.get("block.x", tuple(residual.shape), rt.dtype)
+            rt.ops.to_activation(residual, x)
+        kept, ctx.residual, ctx.takes_normed_deltas = ctx.residual, None, True
+        try:
+            mixed = self.mixer.forward(x, ctx, cache, state, writes_cache)
+            ctx.takes_normed_deltas = False
+            x = self.mixer_norm.add_output(residual, mixed, "block.x")
+            if self.feed_forward is not None:
+                x = self.feed_forward_norm.add_output(residual, self.feed_forward.forward(x, ctx), "block.x")
+        finally:
+            ctx.residual, ctx.takes_normed_deltas = kept, False
+        ctx.stream_copy = x
+        return None
+
+
 register_block("prenorm", PreNormBlock)
+register_block("output_norm", OutputNormBlock)
 register_block("sandwich", SandwichBlock)
 register_block("parallel", ParallelBlock)
 register_block("postnorm", PostNormBlock)

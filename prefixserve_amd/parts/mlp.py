@@ -56,10 +56,10 @@ class SwiGLU(FeedForward):
 
 class DenseMLP(FeedForward):
     """down( act(up(x)) ), no gate and no biases. ``activation``: "gelu" (the exact one, with erf),
-    "gelu_tanh", "silu" or "relu". ``names``: "up", "down"."""
+    "gelu_tanh", "silu", "relu" or "squared_relu". ``names``: "up", "down"."""
 
     def __init__(self, hidden_size: int, intermediate_size: int, names: Mapping[str, str], activation: str = "gelu") -> None:
-        if activation not in ("gelu", "gelu_tanh", "silu", "relu"):
+        if activation not in ("gelu", "gelu_tanh", "silu", "relu", "squared_relu"):
             raise ValueError(f"the feed-forward's activation {activation!r} is not implemented")
         self.activation = activation
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)

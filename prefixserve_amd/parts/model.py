@@ -18,6 +18,7 @@ from . import moe as _moe  # noqa: F401
 from . import norm as _norm  # noqa: F401
 from . import parallel as _parallel  # noqa: F401
 from . import recurrent as _recurrent  # noqa: F401
+from . import retention as _retention  # noqa: F401
 from . import rope as _rope  # noqa: F401
 from . import ssm as _ssm  # noqa: F401
 from . import stream as _stream  # noqa: F401
@@ -51,6 +52,12 @@ class DecoderModel:
         self.embedding_transforms = [make("transform", ps.kind, **sizes, **ps.params) for ps in spec.embedding_transforms]
         # A constant in front of everything else is the gather's own factor.
         self.embedding_factor = getattr(self.embedding_transforms[0], "embedding_factor", None) if self.embedding_transforms else None
+        for tr in self.embedding_transforms[1:]:
+            if tr.gather is not None or tr.state_need() is not None:
+                raise ValueError("a transform that does the gather or keeps state comes first behind the token table")
+        # The block of the first run reads the stream's copy in the activation dtype: a gather may write it as well.
+        self.gather_copies = bool(self.blocks) and getattr(self.blocks[spec.order[0].layer], "reads_stream_copy", False) \
+            and len(self.embedding_transforms) == 1
         self.logit_transforms = [make("transform", ps.kind, **sizes, **ps.params) for ps in spec.logit_transforms]
         self.stream_transforms = {name: make("transform", ps.kind, **sizes, **ps.params)
                                   for name, ps in spec.stream_transforms.items()}
@@ -137,8 +144,11 @@ class DecoderModel:
         return out
 
     def state_needs(self) -> dict[int, StateNeed]:
-        """index into ``spec.order`` -> fixed-size per-request state its mixer keeps."""
+        """index into ``spec.order`` -> fixed-size per-request state its mixer keeps; -1: that of the first transform
+        behind the token table."""
         needs: dict[int, StateNeed] = {}
+        if self.embedding_transforms and self.embedding_transforms[0].state_need() is not None:
+            needs[-1] = self.embedding_transforms[0].state_need()
         for i, run in enumerate(self.spec.order):
             need = self._block_state_need(self.blocks[run.layer])
             if need is not None:
@@ -154,6 +164,8 @@ class DecoderModel:
 
     def state_in_graphs(self) -> bool:
         """Whether every part that keeps state lets a captured decode step update it."""
+        if any(tr.state_need() is not None and not tr.state_in_graphs for tr in self.embedding_transforms[:1]):
+            return False
         return all(getattr(blk, "state_in_graphs", blk.mixer.state_in_graphs) for blk in self.blocks
                    if self._block_state_need(blk) is not None)
 
@@ -183,17 +195,24 @@ class DecoderModel:
                 residual = streams[0]
             else:
                 streams = residual = ws.get("residual", (t, s.hidden_size), torch.float32)
-            if self.embedding_factor is not None:
+            copy = None
+            first = self.embedding_transforms[0] if self.embedding_transforms else None
+            if first is not None and first.gather is not None:
+                if self.gather_copies and rt.dtype != torch.float32:
+                    copy = ws.get("block.x", (t, s.hidden_size), rt.dtype)
+                first.gather(ctx.token_ids, self.embedding, residual, ctx, self.states.get(-1), copy)
+            elif self.embedding_factor is not None:
                 ops.embed(ctx.token_ids, self.embedding, residual, factor=self.embedding_factor)
             else:
                 ops.embed(ctx.token_ids, self.embedding, residual)
-            for tr in self.embedding_transforms[0 if self.embedding_factor is None else 1:]:
+            done = first is not None and (first.gather is not None or self.embedding_factor is not None)
+            for tr in self.embedding_transforms[1 if done else 0:]:
                 tr.apply(residual, ctx, None)
             if s.streams > 1:
                 streams[1:].copy_(residual.unsqueeze(0).expand(s.streams - 1, t, s.hidden_size))
             ctx.residual = residual
             ctx.residual_scale = None
-            ctx.stream_copy = None           # a context may be stepped twice (a graph's eager run, then its capture)
+            ctx.stream_copy = copy           # a context may be stepped twice (a graph's eager run, then its capture)
             if self.keeps_embedding_output:
                 ctx.embedding_output = ws.get("embedding.output", (t, s.hidden_size), torch.float32)
                 ctx.embedding_output.copy_(residual)

@@ -12,15 +12,25 @@ if TYPE_CHECKING:
     from prefixserve_amd.engine.batch import StepContext
 
 
+# How a router scores: the code the kernels take.
+SCORES = {"sigmoid": 0, "softmax_of_chosen": 1, "softmax": 2}
+
+
 class RoutedExperts(FeedForward):
     """``num_experts`` feed-forwards of inner size ``intermediate_size`` without biases, of
     which every token uses ``top_k``.
 
     Router: z = W_r x (+ a bias, ``router_bias``) in 32-bit; the ``top_k`` largest are taken (the
     lower index among equals). ``score`` "sigmoid": the weights are sigmoid(z) as they are, not
-    renormalized; "softmax_of_chosen": the softmax over the chosen z alone. ``groups`` = {"count": G, "keep": k}
-    (sigmoid scores): the experts form G equal groups of neighbours, a group's score is the sum of its two
-    largest scores, and only experts of the k best groups can be chosen. ``weight_scale`` multiplies the weights.
+    renormalized; "softmax_of_chosen": the softmax over the chosen z alone; "softmax": the softmax over all z.
+    ``choice_bias`` (with "softmax"): a learned number per expert (name "correction") that is added to its score for the
+    choice, not for its weight. ``groups`` = {"count": G, "keep": k} (not with "softmax_of_chosen"): the experts form G
+    equal groups of neighbours, a group's score is the sum of its two largest scores (``group_score`` "top2") or its
+    largest ("max"), as the choice sees them, and only experts of the k best groups can be chosen. ``weight_scale``
+    multiplies the weights.
+
+    ``identity``: the router has that many rows more than there are experts, and the last ``identity`` choices are
+    identity experts: their output is the token itself times the weight. They count for ``top_k`` and in the groups.
 
     ``weight_on`` "input": the weight multiplies the expert's input, the output is the sum over
     the chosen experts of expert(w x), which is not w expert(x) when the expert clamps; "output": the
@@ -38,7 +48,7 @@ class RoutedExperts(FeedForward):
     hidden]`` that the norm behind adds up in ascending order, so a token's sum does not depend on
     what else is in the step; in a bfloat16 step so small that the products add into the residual stream
     themselves (``ops.fuses_norm``) the experts do so too. ``names``: "router" ("router_bias"), "gate"/"up"/"down" with ``{e}``
-    for the expert, "shared_gate"/"shared_up"/"shared_down" ("shared_scale": the [1, hidden] row w)."""
+    for the expert, "shared_gate"/"shared_up"/"shared_down" ("shared_scale": the [1, hidden] row w; "correction")."""
 
     takes_residual_scale = True
 
@@ -46,26 +56,35 @@ class RoutedExperts(FeedForward):
                  names: Mapping[str, str], limit: float | None = None, gate_alpha: float = 1.702, up_shift: float = 1.0,
                  score: str = "sigmoid", renormalize: bool = False, weight_on: str = "input",
                  router_bias: bool = False, shared: Mapping[str, object] | None = None, expert: str = "gated",
-                 groups: Mapping[str, int] | None = None, weight_scale: float = 1.0) -> None:
-        if score not in ("sigmoid", "softmax_of_chosen") or renormalize or weight_on not in ("input", "output"):
-            raise ValueError("the router kernels score with a sigmoid (scores kept as weights) or with the softmax over the "
+                 groups: Mapping[str, int] | None = None, weight_scale: float = 1.0, choice_bias: bool = False,
+                 group_score: str = "top2", identity: int = 0) -> None:
+        if score not in SCORES or renormalize or weight_on not in ("input", "output"):
+            raise ValueError("the router kernels score with a sigmoid or a softmax (scores kept as weights) or with the softmax over the "
                              f"chosen logits, on the experts' input or output; got score={score!r}, "
                              f"renormalize={renormalize}, weight_on={weight_on!r}")
-        if not 1 <= top_k <= num_experts:
-            raise ValueError(f"top_k {top_k} of {num_experts} experts")
+        choices = num_experts + identity
+        if num_experts < 1 or identity < 0 or not 1 <= top_k <= choices:
+            raise ValueError(f"top_k {top_k} of {num_experts} experts and {identity} identity experts")
+        if choice_bias and score != "softmax":
+            raise ValueError("a correction of the choice goes with the softmax over all experts")
+        if identity and weight_on != "output":
+            raise ValueError("identity experts' weights multiply the output")
+        if group_score not in ("top2", "max"):
+            raise ValueError(f"a group's score is that of its two largest or of its largest, got {group_score!r}")
         if expert not in ("gated", "squared_relu"):
             raise ValueError(f"experts are gated or squared ReLU without a gate, got {expert!r}")
         if groups is not None:
             count, keep = int(groups["count"]), int(groups["keep"])
-            if score != "sigmoid" or not 1 <= count <= 256 or num_experts % count or not 1 <= keep <= count \
-                    or top_k > keep * (num_experts // count):
-                raise ValueError(f"{num_experts} experts in {count} groups of which {keep} are kept, {top_k} chosen, score {score!r}")
+            if score == "softmax_of_chosen" or not 1 <= count <= 256 or choices % count or not 1 <= keep <= count \
+                    or top_k > keep * (choices // count):
+                raise ValueError(f"{choices} experts in {count} groups of which {keep} are kept, {top_k} chosen, score {score!r}")
         self.hidden_size, self.num_experts, self.top_k = int(hidden_size), int(num_experts), int(top_k)
         self.intermediate_size = int(intermediate_size)
         self.names = dict(names)
         self.limit = float("inf") if limit is None else float(limit)
         self.gate_alpha, self.up_shift = float(gate_alpha), float(up_shift)
-        self.router_mode = 0 if score == "sigmoid" else 1
+        self.router_mode = SCORES[score]
+        self.choice_bias, self.identity, self.choices = bool(choice_bias), int(identity), int(choices)
         self.weight_on_output = weight_on == "output"
         self.router_bias = bool(router_bias)
         self.shared_size = None if shared is None else int(shared["intermediate_size"])
@@ -77,9 +96,13 @@ class RoutedExperts(FeedForward):
             self.route_options["mode"] = self.router_mode
         if groups is not None:
             self.route_options.update(groups=count, keep=keep)
+            if group_score == "max":
+                self.route_options["group_max"] = True
         if weight_scale != 1.0:
             self.route_options["factor"] = float(weight_scale)
         self.expert_options: dict[str, object] = {}
+        if self.identity:
+            self.route_options["identity"] = self.expert_options["identity"] = self.identity
         if self.weight_on_output:
             self.expert_options["weight_on_output"] = True
         if expert != "gated":
@@ -87,9 +110,11 @@ class RoutedExperts(FeedForward):
 
     def weights(self) -> dict[str, WeightWant]:
         h, f, n = self.hidden_size, self.intermediate_size, self.names
-        want = {n["router"]: WeightWant((self.num_experts, h))}
+        want = {n["router"]: WeightWant((self.choices, h))}
         if self.router_bias:
-            want[n["router_bias"]] = WeightWant((self.num_experts,), "bias")
+            want[n["router_bias"]] = WeightWant((self.choices,), "bias")
+        if self.choice_bias:
+            want[n["correction"]] = WeightWant((self.choices,), "offset")
         for e in range(self.num_experts):
             if self.expert == "gated":
                 want[n["gate"].format(e=e)] = WeightWant((f, h))
@@ -114,6 +139,8 @@ class RoutedExperts(FeedForward):
         self.b_router = None
         if self.router_bias:
             self.b_router = tensors[n["router_bias"]].to(device=rt.device, dtype=torch.float32).contiguous()
+        if self.choice_bias:
+            self.route_options["correction"] = tensors[n["correction"]].to(device=rt.device, dtype=torch.float32).contiguous()
         # Per expert the rows of gate (where there is one), then of up: [E, 2F or F, H]; and down [E, H, F].
         first = ("gate", "up") if self.expert == "gated" else ("up",)
         self.w_in = rt.ops.prepare_matrix(torch.stack([torch.cat([tensors[n[which].format(e=e)] for which in first], dim=0)

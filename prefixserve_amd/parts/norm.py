@@ -6,7 +6,7 @@ from typing import Mapping
 
 import torch
 
-from .base import Norm, NormedRows, Runtime, WeightWant, register_norm
+from .base import Norm, NormedDeltas, NormedRows, Runtime, WeightWant, register_norm
 
 
 class RMSNorm(Norm):
@@ -39,6 +39,7 @@ class RMSNorm(Norm):
         if self.unit_offset:
             w = 1.0 + w.to(torch.float32)
         self.weight = w.to(rt.device).contiguous()
+        self._weight32: torch.Tensor | None = None       # made when a norm on an output asks for it
 
     def weight_bytes(self) -> int:
         return self.weight.numel() * self.weight.element_size()
@@ -72,6 +73,15 @@ class RMSNorm(Norm):
         rt = self.rt
         out = None if rt.dtype == torch.float32 else rt.workspace.get(out_name, tuple(residual.shape), rt.dtype)
         rt.ops.scaled_add_rmsnorm(residual, delta, float(alpha), self.weight, self.eps, out)
+        return residual if out is None else out
+
+
+    def add_output(self, residual: torch.Tensor, delta: "torch.Tensor | NormedDeltas", out_name: str) -> torch.Tensor:
+        rt = self.rt
+        if self._weight32 is None:
+            self._weight32 = self.weight.to(torch.float32).contiguous()
+        out = None if rt.dtype == torch.float32 else rt.workspace.get(out_name, tuple(residual.shape), rt.dtype)
+        rt.ops.output_norm(residual, delta, self._weight32, self.eps, out)
         return residual if out is None else out
 
 

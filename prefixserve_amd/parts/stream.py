@@ -7,7 +7,7 @@ from typing import TYPE_CHECKING, Mapping
 
 import torch
 
-from .base import Runtime, Transform, WeightWant, register_transform
+from .base import Runtime, StateNeed, Transform, WeightWant, register_transform
 
 if TYPE_CHECKING:
     from prefixserve_amd.engine.batch import StepContext
@@ -107,6 +107,39 @@ class SinusoidalPositions(Transform):
         self.rt.ops.add_sinusoid(t, ctx.positions, self.freq)
 
 
+class BigramEmbedding(Transform):
+    """t <- t + bigram[(p * mul_prev + c * mul_cur) mod buckets] with c the row's token and p the one in front of it; a
+    sequence's first token takes the table's last row, number ``buckets``. It is the gather itself (the token table's row
+    and the bigram's in one kernel, sums in 32-bit) and keeps each request's last token in a slot, as token + 1 (0: none).
+    ``name``: the table [buckets + 1, hidden]."""
+
+    state_in_graphs = True
+
+    def __init__(self, hidden_size: int, vocab_size: int, buckets: int, mul_prev: int, mul_cur: int, name: str) -> None:
+        self.hidden_size, self.buckets, self.name = int(hidden_size), int(buckets), name
+        self.mul_prev, self.mul_cur = int(mul_prev), int(mul_cur)
+        if self.buckets < 1 or (abs(self.mul_prev) + abs(self.mul_cur)) * int(vocab_size) >= 1 << 62:
+            raise ValueError(f"{buckets} buckets, multipliers {mul_prev} and {mul_cur}")
+
+    def weights(self) -> dict[str, WeightWant]:
+        return {self.name: WeightWant((self.buckets + 1, self.hidden_size), "embedding")}
+
+    def state_need(self) -> StateNeed:
+        return StateNeed((1,), torch.int32)
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
+        super().bind(tensors, rt)
+        self.table = rt.ops.prepare_matrix(tensors[self.name], rt)
+
+    def gather(self, ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, ctx: "StepContext", state: torch.Tensor,
+               copy: torch.Tensor | None) -> None:
+        self.rt.ops.embed_bigram(ids, table, self.table, out, copy, state, ctx, self.mul_prev, self.mul_cur)
+
+    def apply(self, t: torch.Tensor, ctx: "StepContext", rows: torch.Tensor | None) -> None:
+        raise ValueError("the bigram embedding is the first transform behind the token table: it does the gather itself")
+
+
+register_transform("bigram_embedding", BigramEmbedding)
 register_transform("scale", ScaleStream)
 register_transform("sinusoidal_positions", SinusoidalPositions)
 register_transform("reentry", StreamReentry)
