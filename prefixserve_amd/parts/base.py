@@ -257,6 +257,8 @@ class Mixer(Part):
     # run's state; a container (a block with state of its own, a mixer made of several) lays its
     # parts' states side by side and sets this before the first step.
     state_base = 0
+    # ... and the multiple of numbers it begins at (and a slot's row takes).
+    state_align = 1
 
     # True: the mixer reads x through one input matrix alone and can be handed the product: ``input_matrix(tensors)`` gives
     # the matrix [n, hidden] (on the host) and ``forward_rows(rows, col, ctx, cache, state, writes_cache)`` runs from

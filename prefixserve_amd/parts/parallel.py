@@ -18,7 +18,7 @@ class ParallelMixers(Mixer):
     with its own output matrix, and the weighted sum (32-bit) is what the layer adds. ``left``
     and ``right`` are ``PartSpec``s of any registered mixers; their weight names are theirs. At
     most one of them may keep keys in pages; their fixed-size states lie side by side in the
-    run's slot, the left one's first, each from a multiple of four numbers on.
+    run's slot, the left one's first, each from a multiple of what either asks for (``state_align``) on.
 
     ``out_norms`` = {"left": name, "right": name, "eps": e, "scale": s}: each output is divided by its root mean square over
     the width and multiplied by a weight first; the result is s times their sum, formed in 32-bit by the kernel that adds it
@@ -43,12 +43,13 @@ class ParallelMixers(Mixer):
         self._place()
 
     def _sizes(self) -> list[int]:
-        out = []
+        out, align = [], max(m.state_align for m in (self.left, self.right))
         for m in (self.left, self.right):
             need = m.state_need()
             if need is not None and need.dtype != torch.float32:
                 raise ValueError("states laid side by side must be 32-bit")
-            out.append(0 if need is None else -(-int(torch.Size(need.shape).numel()) // 4) * 4)
+            size = 0 if need is None else int(torch.Size(need.shape).numel())
+            out.append(-(-size // align) * align)
         return out
 
     def _place(self) -> None:

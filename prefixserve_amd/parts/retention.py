@@ -31,6 +31,7 @@ class Retention(Mixer):
     not depend on the token, a portion runs in pieces side by side on the matrix cores. ``names``: "q", "k", "v", "gate", "o"."""
 
     state_in_graphs = True
+    state_align = 4                  # the kernels read and write four values of the state at a time
     takes_input_rows = True
 
     def __init__(self, hidden_size: int, positions: Mapping[str, PositionEncoding], num_heads: int, head_dim: int, value_dim: int,

@@ -13,7 +13,7 @@ import contextlib
 
 import torch
 
-from prefixserve_amd.parts.base import ScaledDelta
+from prefixserve_amd.parts.base import NormedDeltas, ScaledDelta
 
 PAGE = 16
 
@@ -244,29 +244,35 @@ class EmulatedOps:
             vals = raw_keys if values_from_keys else qkv[:, (hq + hkv) * d:].view(t, hkv, d)
             kv[:, 1].view(kv.shape[0], hkv, d, PAGE)[page, :, :, off] = vals
 
-    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode=0, groups=0, keep=0, factor=1.0) -> None:
+    def moe_route(self, x, w_router, chosen, weight, w_router_act=None, bias=None, mode=0, groups=0, keep=0, factor=1.0,
+                  group_max=False, correction=None, identity=0) -> None:
         z = x.float() @ w_router.float().T
         if bias is not None:
             z = z + bias
-        s = torch.sigmoid(z) if mode == 0 else z
+        score = s = torch.sigmoid(z) if mode == 0 else torch.softmax(z, dim=-1) if mode == 2 else z
+        if correction is not None:
+            s = s + correction
         if groups:
             per = s.view(s.shape[0], groups, -1)
-            sums = per.topk(min(2, per.shape[2]), dim=-1).values.sum(-1)
+            sums = per.topk(min(1 if group_max else 2, per.shape[2]), dim=-1).values.sum(-1)
             best = torch.argsort(-sums, dim=-1, stable=True)[:, :keep]
             allowed = torch.zeros_like(sums, dtype=torch.bool).scatter_(1, best, True)
             s = per.masked_fill(~allowed[:, :, None], float("-inf")).reshape(s.shape)
         order = torch.argsort(-s, dim=-1, stable=True)[:, : chosen.shape[1]]
         chosen.copy_(order.to(torch.int32))
-        picked = torch.gather(s, 1, order)
-        weight.copy_(factor * (picked if mode == 0 else torch.softmax(picked, dim=-1)))
+        picked = torch.gather(score, 1, order)
+        weight.copy_(factor * (torch.softmax(picked, dim=-1) if mode == 1 else picked))
 
     def moe_experts(self, x, chosen, weight, w_in, w_down, act, out, gate_alpha, limit, up_shift,
-                    weight_on_output=False, kind="gated", residual=None, col_scale=None) -> None:
+                    weight_on_output=False, kind="gated", residual=None, col_scale=None, identity=0) -> None:
         t, k = chosen.shape
         f = w_down.shape[2]
         for i in range(t):
             for j in range(k):
                 e = int(chosen[i, j])
+                if e >= w_down.shape[0]:
+                    out[j, i] = weight[i, j] * x[i].float()
+                    continue
                 h = x[i].float() * (1.0 if weight_on_output else weight[i, j])
                 gu = w_in[e].float() @ h
                 if kind == "gated":
@@ -394,7 +400,7 @@ class EmulatedOps:
 
     def activation(self, x, kind) -> None:
         f = {"gelu": torch.nn.functional.gelu, "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh"),
-             "silu": torch.nn.functional.silu, "relu": torch.relu}[kind]
+             "silu": torch.nn.functional.silu, "relu": torch.relu, "squared_relu": lambda z: torch.relu(z).square()}[kind]
         x.copy_(f(x.float()).to(x.dtype))
 
     def gated_group_norm(self, y, x, x_col, skip, heads, gate_rows, gate_col, weight, groups, eps, out) -> None:
@@ -485,7 +491,7 @@ class EmulatedOps:
             out[row] = o.reshape(hq * d).to(out.dtype)
 
     def paged_attention(self, qkv, out, kv, ctx, group, hq, hkv, d, scale, window, exact_weights=False, sink=None,
-                        dist_bias=None, keep_first=0, pooled=None, head_gate=None) -> None:
+                        dist_bias=None, keep_first=0, pooled=None, head_gate=None, out_gate=None) -> None:
         if keep_first or pooled is not None or head_gate is not None:
             return self._masked_attention(qkv, out, kv, ctx, group, hq, hkv, d, scale, window, keep_first, pooled, head_gate)
         g = ctx.groups[group]
@@ -518,7 +524,93 @@ class EmulatedOps:
             probs = torch.softmax(scores, dim=-1)
             if sink is not None:
                 probs = probs[..., :-1]
-            o[t0:t1] = torch.matmul(probs, vals.transpose(0, 1)).transpose(0, 1).to(out.dtype)
+            y = torch.matmul(probs, vals.transpose(0, 1)).transpose(0, 1)
+            if out_gate is not None:
+                rows, col = out_gate
+                y = y * torch.sigmoid(rows[t0:t1, col: col + hq * d].float().view(-1, hq, d))
+            o[t0:t1] = y.to(out.dtype)
+
+    # ----------------------------------------------- a bigram table, norms on outputs, short convolutions, retention
+
+    def embed_bigram(self, ids, table, bigram, out, copy, state, ctx, mul_prev, mul_cur) -> None:
+        starts, buckets = ctx.item_start.tolist(), bigram.shape[0] - 1
+        for i in range(ctx.num_items):
+            slot = int(ctx.slots[i])
+            before = int(state[slot, 0]) - 1
+            for t in range(starts[i], starts[i + 1]):
+                cur = int(ids[t])
+                row = buckets if before < 0 else (before * mul_prev + cur * mul_cur) % buckets
+                out[t] = table[cur].float() + bigram[row].float()
+                before = cur
+            state[slot, 0] = before + 1
+        if copy is not None:
+            copy.copy_(out.to(copy.dtype))
+
+    def output_norm(self, residual, delta, weight, eps, out) -> None:
+        def normed(y, e):
+            return y * torch.rsqrt((y * y).mean(-1, keepdim=True) + e)
+
+        if isinstance(delta, NormedDeltas):
+            y = delta.scale * sum(normed(self._whole(d), delta.eps) * w for d, w in delta.parts)
+        else:
+            y = self._whole(delta)
+        residual.add_(normed(y, eps) * weight)
+        if out is not None:
+            out.copy_(residual.to(out.dtype))
+
+    def qkv_conv_append(self, rows, col, conv_w, hq, hkv, d, positions, table, norm_dim, norm_eps, q_weight, k_weight, q_out, kv,
+                        write_slot, state, state_offset, ctx) -> None:
+        taps, channels = conv_w.shape
+        t, keep = q_out.shape[0], taps - 1
+        y = torch.empty((t, channels))
+        starts = ctx.item_start.tolist()
+        for i in range(ctx.num_items):
+            t0, t1 = starts[i], starts[i + 1]
+            v = rows[t0:t1, col: col + channels].float()
+            if keep:
+                saved = state[int(ctx.slots[i]), state_offset: state_offset + keep * channels].view(keep, channels)
+                v = torch.cat([saved, v], dim=0)
+                saved.copy_(v[-keep:].clone())
+            y[t0:t1] = sum(conv_w[j] * v[j: j + t1 - t0] for j in range(taps))
+        heads = y[:, : (hq + hkv) * d].view(t, hq + hkv, d)
+        if norm_dim:
+            heads = heads * torch.rsqrt((heads * heads).sum(-1, keepdim=True) / norm_dim + norm_eps)
+        parts = [heads[:, :hq], heads[:, hq:]]
+        for k, w in enumerate((q_weight, k_weight)):
+            if w is not None:
+                parts[k] = parts[k] * w
+        if table is not None:
+            cos, sin = (table[positions.long()][..., k][:, None, :] for k in (0, 1))
+            parts = [torch.cat([x[..., : d // 2] * cos - x[..., d // 2:] * sin, x[..., d // 2:] * cos + x[..., : d // 2] * sin], dim=-1)
+                     for x in parts]
+        q_out.copy_(parts[0].reshape(t, hq * d).to(q_out.dtype))
+        if kv is not None:
+            page, off = (write_slot // PAGE).long(), (write_slot % PAGE).long()
+            kv[:, 0].view(kv.shape[0], hkv, PAGE, d)[page, :, off, :] = parts[1].to(kv.dtype)
+            kv[:, 1].view(kv.shape[0], hkv, d, PAGE)[page, :, :, off] = y[:, (hq + hkv) * d:].view(t, hkv, d).to(kv.dtype)
+
+    def retention_powers(self) -> int:
+        return 2
+
+    def retention(self, rows, q_col, k_col, v_col, g_col, table, powers, k_scale, state, state_offset, ctx, heads, dim_p, vdim_p, vdim,
+                  eps, out) -> None:
+        t = out.shape[0]
+        q, k = (rows[:, c: c + heads * dim_p].float().view(t, heads, dim_p).clone() for c in (q_col, k_col))
+        if table is not None:
+            r = 2 * table.shape[1]
+            for x in (q, k):
+                x[..., :r] = self._turn(x[..., :r].clone(), table, ctx.positions, True)
+        k = k * k_scale
+        v, g = (rows[:, c: c + heads * vdim_p].float().view(t, heads, vdim_p) for c in (v_col, g_col))
+        o = torch.empty((t, heads, vdim_p))
+        starts = ctx.item_start.tolist()
+        for i in range(ctx.num_items):
+            s = state[int(ctx.slots[i]), state_offset: state_offset + heads * dim_p * vdim_p].view(heads, dim_p, vdim_p)
+            for n in range(starts[i], starts[i + 1]):
+                s.copy_(powers[:, 1, None, None] * s + k[n][:, :, None] * v[n][:, None, :])
+                o[n] = torch.einsum("hdv,hd->hv", s, q[n])
+        o = o * torch.rsqrt((o * o).sum(-1, keepdim=True) / vdim + eps) * torch.nn.functional.silu(g)
+        out.copy_(o.reshape(t, heads * vdim_p).to(out.dtype))
 
     def argmax(self, logits, out) -> None:
         out.copy_(torch.argmax(logits, dim=-1).to(out.dtype))
