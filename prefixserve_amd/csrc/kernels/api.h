@@ -384,13 +384,13 @@ int psamd_qkv_conv_append(void* stream, const void* in, int act_dtype, int64_t i
                           const int32_t* tok_item, const int32_t* item_start, const int32_t* slots, int64_t tokens, int items);
 
 // Retention (linear attention with a fixed decay per head), gated and normalized per head: see retention.hip. rows: q, k
-// (heads of dim_p), v, gate (heads of vdim_p) at their columns; table float [pos][rot / 2][2]; powers float [heads]
+// (heads of dim_p), v, gate (heads of vdim_p) at their columns; table float [pos][dim_p / 2][2]; powers float [heads]
 // [psamd_retention_powers()]: powers of the heads' decays from 0 on; state float, of slot s at state + s * state_row, [heads]
 // [dim_p][vdim_p]; pf_tiles / pf_blocks: the step's tiles of 32 tokens and runs of four of them; dec_items: its single-token
 // items; sums: room for n_blocks * heads * dim_p * vdim_p floats; out [tokens][heads * vdim_p].
 int psamd_retention_powers(void);
 int psamd_retention(void* stream, const void* rows, int act_dtype, int64_t row, int q_col, int k_col, int v_col, int g_col,
-                    const int32_t* positions, const float* table, int rot, const float* powers, float k_scale, float* state,
+                    const int32_t* positions, const float* table, const float* powers, float k_scale, float* state,
                     int64_t state_row, const int32_t* item_start, const int32_t* slots, const int32_t* pf_tiles, int n_tiles,
                     int tile_tokens, const int32_t* pf_blocks, int n_blocks, const int32_t* dec_items, int n_dec, float* sums,
                     int heads, int dim_p, int vdim_p, int vdim, float eps, void* out);

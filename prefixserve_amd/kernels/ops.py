@@ -125,7 +125,7 @@ _SIGNATURES = {
     "psamd_qkv_conv_append": [_vp, _vp, _i32, _i64, _vp, _i32, _i32, _i32, _i32, _vp, _vp, _i32, _f32, _vp, _vp, _vp, _vp, _vp,
                               _vp, _i64, _vp, _vp, _vp, _i64, _i32],
     "psamd_retention_powers": [],
-    "psamd_retention": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _vp, _vp, _i32, _vp, _f32, _vp, _i64, _vp, _vp, _vp, _i32,
+    "psamd_retention": [_vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _vp, _vp, _vp, _f32, _vp, _i64, _vp, _vp, _vp, _i32,
                         _i32, _vp, _i32, _vp, _i32, _vp, _i32, _i32, _i32, _i32, _f32, _vp],
     "psamd_output_norm": [_vp, _vp, _vp, _i32, _i32, _i64, _vp, _vp, _i32, _i32, _i64, _vp, _f32, _f32, _vp, _f32, _vp, _i32, _i64,
                           _i32],
@@ -1009,7 +1009,7 @@ class HipOps:
     def retention(self, rows, q_col: int, k_col: int, v_col: int, g_col: int, table, powers, k_scale: float, state, state_offset: int, ctx,
                   heads: int, dim_p: int, vdim_p: int, vdim: int, eps: float, out) -> None:
         """Linear attention with a fixed decay per head over each item's tokens from its state slot: q, k rotated (``table`` float32
-        [pos, rot/2, 2], pairs (i, i + rot/2) of the first rot dimensions; None: not), k times ``k_scale``, S <- decay S + k v^T, o = S^T q,
+        [pos, dim_p/2, 2], pairs (i, i + dim_p/2); (1, 0) where nothing turns), k times ``k_scale``, S <- decay S + k v^T, o = S^T q,
         out = o / sqrt(mean(o^2) + eps) * silu(gate), per head, the mean over ``vdim``. ``rows`` hold q and k (heads of ``dim_p``), v and gate
         (heads of ``vdim_p``) from their columns on, sizes padded with zeros to multiples of 16. ``powers`` float32 [heads,
         ``retention_powers()``]. The state of a head is float32 [dim_p, vdim_p], heads one behind the other from ``state_offset`` on."""
@@ -1017,10 +1017,7 @@ class HipOps:
         self._need(rows.dim() == 2 and rows.is_contiguous() and rows.shape[0] == t == ctx.num_tokens, "retention: rows")
         self._need(out.dtype == rows.dtype and out.shape == (t, heads * vdim_p) and out.is_contiguous(), "retention: out")
         self._need(powers.dtype == torch.float32 and powers.shape == (heads, self.retention_powers()) and powers.is_contiguous(), "retention: powers")
-        rot = 0
-        if table is not None:
-            self._need(table.dtype == torch.float32 and table.dim() == 3 and table.shape[2] == 2 and table.is_contiguous(), "retention: table")
-            rot = 2 * table.shape[1]
+        self._need(table.dtype == torch.float32 and table.shape[1:] == (dim_p // 2, 2) and table.is_contiguous(), "retention: table")
         self._need(state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous() and 0 <= state_offset
                    and state_offset + heads * dim_p * vdim_p <= state.shape[1], "retention: the state")
         n_blocks = int(ctx.num_prefill_blocks)
@@ -1032,7 +1029,7 @@ class HipOps:
             self._need(n_blocks <= most, "retention: more runs than tokens and slots allow")
             sums = self.ws.get("retention.sums", (most * heads * dim_p * vdim_p,), torch.float32)
         self._ok(self.lib.psamd_retention(
-            self._stream(), rows.data_ptr(), _code(rows.dtype), rows.shape[1], q_col, k_col, v_col, g_col, ctx.positions.data_ptr(), _ptr(table), rot,
+            self._stream(), rows.data_ptr(), _code(rows.dtype), rows.shape[1], q_col, k_col, v_col, g_col, ctx.positions.data_ptr(), table.data_ptr(),
             powers.data_ptr(), float(k_scale), state.data_ptr() + 4 * state_offset, state.shape[1], ctx.item_start.data_ptr(),
             ctx.slots.data_ptr(), ctx.pf_tiles.data_ptr(), ctx.num_prefill_tiles, self.PREFILL_TILE_Q, ctx.pf_blocks.data_ptr(), n_blocks,
             ctx.dec_items.data_ptr(), ctx.num_decode, _ptr(sums), heads, dim_p, vdim_p, vdim, float(eps), out.data_ptr()))

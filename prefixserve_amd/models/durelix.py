@@ -15,6 +15,7 @@ from __future__ import annotations
 from prefixserve_amd.config.durelix import MAX_POSITION, DenseFeedForward, DurelixConfig, Rotary
 from prefixserve_amd.config.registry import register_architecture
 from prefixserve_amd.parts.attention import slot_size
+from prefixserve_amd.parts.retention import padded
 from prefixserve_amd.parts.spec import LayerRun, LayerSpec, ModelSpec, PartSpec
 
 ATTENTION_NAMES = {"q": "mix.left.q", "k": "mix.left.k", "v": "mix.left.v", "o": "mix.left.o", "q_norm": "mix.left.q.norm",
@@ -37,13 +38,12 @@ def build_durelix_spec(cfg: DurelixConfig) -> ModelSpec:
     positions: dict[str, PartSpec] = {}
     by_params: dict[tuple, str] = {}
 
-    def rotation(rot: Rotary | None, head_dim: int) -> dict[str, str]:
+    def rotation(rot: Rotary | None, head_dim: int) -> str:
         """The encoding for heads of ``head_dim`` slots; equal rotations share one table."""
-        if rot is None or rot.dims == 0:
-            return {}
-        name = by_params.setdefault((head_dim, rot.dims, rot.base), f"rot{len(by_params)}")
-        positions[name] = PartSpec("rope", {"head_dim": head_dim, "theta": rot.base, "rotary_dim": rot.dims})
-        return {"position": name}
+        dims, base = (rot.dims, rot.base) if rot is not None else (0, 1.0)
+        name = by_params.setdefault((head_dim, dims, base), f"rot{len(by_params)}")
+        positions[name] = PartSpec("rope", {"head_dim": head_dim, "theta": base, "rotary_dim": dims})
+        return name
 
     for i, layer in enumerate(cfg.layers):
         a, r = layer.mixer.left, layer.mixer.right
@@ -51,11 +51,11 @@ def build_durelix_spec(cfg: DurelixConfig) -> ModelSpec:
             "num_heads": a.heads, "num_kv_heads": a.kv_heads, "head_dim": a.dim, "value_dim": a.vdim, "names": ATTENTION_NAMES,
             "scale": a.scale, "window": a.window, "qk_norm_eps": cfg.norm_eps, "qk_norm_weights": True, "norm_first": True,
             "pairs": "neighbours", "conv_taps": a.conv, "sink": True, "out_gate": True, "exact_weights": True,
-            **rotation(a.rot, slot_size(a.dim, a.vdim)),
+            "position": rotation(a.rot, slot_size(a.dim, a.vdim)),
         })
         right = PartSpec("retention", {
             "num_heads": r.heads, "head_dim": r.dim, "value_dim": r.vdim, "decays": r.decay, "names": RETENTION_NAMES,
-            "norm_eps": cfg.norm_eps, **rotation(r.rot, r.rot.dims if r.rot is not None else 0),
+            "norm_eps": cfg.norm_eps, "position": rotation(r.rot, padded(r.dim)),
         })
         mixer = PartSpec("parallel_mixers", {
             "left": left, "right": right,

@@ -596,10 +596,7 @@ class EmulatedOps:
                   eps, out) -> None:
         t = out.shape[0]
         q, k = (rows[:, c: c + heads * dim_p].float().view(t, heads, dim_p).clone() for c in (q_col, k_col))
-        if table is not None:
-            r = 2 * table.shape[1]
-            for x in (q, k):
-                x[..., :r] = self._turn(x[..., :r].clone(), table, ctx.positions, True)
+        q, k = (self._turn(x, table, ctx.positions, True) for x in (q, k))
         k = k * k_scale
         v, g = (rows[:, c: c + heads * vdim_p].float().view(t, heads, vdim_p) for c in (v_col, g_col))
         o = torch.empty((t, heads, vdim_p))

@@ -239,15 +239,21 @@ def test_parts_refuse_what_they_do_not_take():
                {"out_gate": True, "qk_norm_eps": 1e-5}, {"out_gate": True, "values_are_keys": True}, {"conv_taps": 2, "qk_bias": True}):
         with pytest.raises(ValueError):
             PagedAttention(**{**base, **kw})
-    for kw in ({"num_heads": 3}, {"head_dim": 300}, {"value_dim": 257}):
+    turns = {name: make("position", "rope", **kw) for name, kw in {
+        "16": {"head_dim": 16, "theta": 9.0, "rotary_dim": 8}, "32": {"head_dim": 32, "theta": 9.0, "rotary_dim": 8},
+        "wide": {"head_dim": 16, "theta": 9.0, "rotary_dim": 10}}.items()}
+    heads = {"hidden_size": 32, "positions": turns, "num_heads": 2, "head_dim": 8, "value_dim": 8, "decays": (0.5, 0.6), "names": names,
+             "norm_eps": 1e-5, "position": "16"}
+    Retention(**heads)
+    for kw in ({"num_heads": 3}, {"head_dim": 300}, {"value_dim": 257}, {"position": "32"}, {"position": "wide"}):
         with pytest.raises(ValueError):
-            Retention(**{"hidden_size": 32, "positions": {}, "num_heads": 2, "head_dim": 8, "value_dim": 8, "decays": (0.5, 0.6), "names": names,
-                         "norm_eps": 1e-5, **kw})
+            Retention(**{**heads, **kw})
     with pytest.raises(ValueError):                              # a hash that would not fit 64 bits
         make("transform", "bigram_embedding", hidden_size=8, vocab_size=1 << 20, buckets=7, mul_prev=1 << 45, mul_cur=1, name="b")
-    left = PartSpec("retention", {"num_heads": 1, "head_dim": 8, "value_dim": 8, "decays": (0.5,), "names": names, "norm_eps": 1e-5})
+    left = PartSpec("retention", {"num_heads": 1, "head_dim": 8, "value_dim": 8, "decays": (0.5,), "names": names, "norm_eps": 1e-5,
+                                   "position": "16"})
     with pytest.raises(ValueError):
-        make("mixer", "parallel_mixers", hidden_size=8, positions={}, left=left, right=left, left_scale=2.0,
+        make("mixer", "parallel_mixers", hidden_size=8, positions=turns, left=left, right=left, left_scale=2.0,
              out_norms={"left": "a", "right": "b", "eps": 1e-5})
 
 
