@@ -231,9 +231,50 @@ def zurolorn_set(size: dict, layers: int, vocab: int) -> dict[str, dict]:
     return {"zurolorn": zurolorn, "gokolix": gokolix, "radivik": radivik, "llama": llama}
 
 
+# Durelix at sizes that resemble real layers, beside the designs with the like parts and Llama: a Fubelorn with one stream and
+# no convolution in front of its sub-layers, every layer attention in the same window beside a matrix memory of the same heads
+# (a linear recurrence with a state of the same size) and a feed-forward without a gate of the same inner size; a Radivik of
+# equal width with gated experts of the same sizes; the Llama decoder of equal size. Four layers: the Durelix's first and last
+# have a dense feed-forward, the two between them experts.
+DURELIX_SIZES = {
+    "durelix-w2048-h32x64-r16x128-ff8192-e32x1024-top8": dict(width=2048, heads=32, kv_heads=8, dim=64, window=1024, ret_heads=16, ret_dim=128,
+                                                              ff=8192, experts=32, identity=4, expert_ff=1024, top=8, groups=4, keep=2),
+    "durelix-w4096-h32x128-r32x128-ff14336-e16x3584-top4": dict(width=4096, heads=32, kv_heads=8, dim=128, window=1024, ret_heads=32, ret_dim=128,
+                                                                ff=14336, experts=16, identity=4, expert_ff=3584, top=4, groups=4, keep=2),
+}
+
+
+def durelix_set(size: dict, layers: int, vocab: int) -> dict[str, dict]:
+    """Name -> config.json of the Durelix and of the models it is set beside. ``layers`` is not used: four layers."""
+    att = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["dim"], "scale": size["dim"] ** -0.5}
+    rot = {"dims": size["dim"], "base": 500000.0}
+    n = size["ret_heads"]
+    left = dict(att, conv=4, mask={"size": size["window"]}, rot=rot)
+    right = {"heads": n, "dim": size["ret_dim"], "vdim": size["ret_dim"], "decay": [1.0 - 2.0 ** (-5.0 - 7.0 * i / n) for i in range(n)],
+             "rot": {"dims": size["ret_dim"], "base": 1e4}}
+    mixer = {"left": left, "right": right}
+    router = {"experts": size["experts"], "top": size["top"]}
+    dense = {"kind": "dense", "ff": size["ff"]}
+    experts = {"kind": "moe", "expert": {"ff": size["expert_ff"]},
+               "router": {**router, "identity": size["identity"], "groups": {"count": size["groups"], "keep": size["keep"]}}}
+    common = {"vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6}}
+    durelix = {"architecture": "Durelix", **common, "embedding": {"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 7}},
+               "layers": [{"type": "parallel", "mixer": mixer, "mlp": mlp} for mlp in (dense, experts, experts, dense)]}
+    memory = {"heads": n, "dim": size["ret_dim"], "vdim": size["ret_dim"], "gate_cap": 15.0}
+    side = {"left": dict(att, mask={"size": size["window"]}, rot=rot), "right": memory, "left_scale": 0.5, "right_scale": 0.5}
+    fubelorn = {"architecture": "Fubelorn", **common, "residual_mult": 0.5, "streams": 1,
+                "layers": [{"type": "parallel_2", "mixer": side, "mlp": dense}] * 4}
+    radivik = {"architecture": "Radivik", **common, "postln_alpha": 2.0,
+               "layers": [{"type": "attention", "mixer": dict(att, rot=rot),
+                           "mlp": {"kind": "moe", "router": router, "expert": {"ff": size["expert_ff"], "limit": 7.0}}}] * 4}
+    llama = dict(LLAMA_1B, vocab_size=vocab, hidden_size=size["width"], intermediate_size=size["ff"], num_hidden_layers=4,
+                 num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=size["dim"], tie_word_embeddings=False)
+    return {"durelix": durelix, "fubelorn": fubelorn, "radivik": radivik, "llama": llama}
+
+
 def compare_designs(args) -> int:
-    """Prefill and decode throughput of another design's layers (Radivik, Gokolix, Larupel, Fubelorn, Zurolorn) beside Llama
-    layers of equal size (Zurolorn: also beside the designs that share its parts), through the same runner and step
+    """Prefill and decode throughput of another design's layers (Radivik, Gokolix, Larupel, Fubelorn, Zurolorn, Durelix) beside
+    Llama layers of equal size (Zurolorn, Durelix: also beside the designs with the like parts), through the same runner and step
     function. One JSON line; the default benchmark is not run."""
     import numpy as np
     import torch
@@ -245,7 +286,11 @@ def compare_designs(args) -> int:
     rng = np.random.default_rng(0)
     vocab, layers = 32000, args.layers or 4
     prompt, batch, context = args.prompt_len, args.batch, args.context
-    if args.compare in ZUROLORN_SIZES or args.compare == "zurolorn":
+    set_of = zurolorn_set
+    if args.compare in DURELIX_SIZES or args.compare == "durelix":
+        design, pair_of, set_of = "durelix", None, durelix_set
+        sizes = DURELIX_SIZES if args.compare == "durelix" else {args.compare: DURELIX_SIZES[args.compare]}
+    elif args.compare in ZUROLORN_SIZES or args.compare == "zurolorn":
         design, pair_of = "zurolorn", None
         sizes = ZUROLORN_SIZES if args.compare == "zurolorn" else {args.compare: ZUROLORN_SIZES[args.compare]}
     elif args.compare in FUBELORN_SIZES or args.compare == "fubelorn":
@@ -317,7 +362,7 @@ def compare_designs(args) -> int:
     with tempfile.TemporaryDirectory(prefix="psamd_compare_") as tmp:
         for name, size in sizes.items():
             if pair_of is None:
-                configs = zurolorn_set(size, layers, vocab)
+                configs = set_of(size, layers, vocab)
             else:
                 other, llama = pair_of(size, layers, vocab)
                 configs = {design: other, "llama": llama}
@@ -375,11 +420,12 @@ def main() -> int:
     ap.add_argument("--model", default=None, help="use this model folder instead of writing random weights")
     ap.add_argument("--shape", choices=sorted(SHAPES), default="llama-3.2-1b", help="layer sizes of the random model")
     ap.add_argument("--compare", choices=sorted(RADIVIK_SIZES) + ["all"] + sorted(GOKOLIX_SIZES) + ["gokolix"] + sorted(LARUPEL_SIZES) + ["larupel"]
-                    + sorted(FUBELORN_SIZES) + ["fubelorn"] + sorted(ZUROLORN_SIZES) + ["zurolorn"], default=None,
-                    help="instead of the benchmark: Radivik, Gokolix, Larupel, Fubelorn or Zurolorn layers of this size ('all': every Radivik "
-                         "size, 'gokolix' / 'larupel' / 'fubelorn' / 'zurolorn': every size of that design) beside Llama layers of equal size (prefill of --prompt-len tokens, "
+                    + sorted(FUBELORN_SIZES) + ["fubelorn"] + sorted(ZUROLORN_SIZES) + ["zurolorn"] + sorted(DURELIX_SIZES) + ["durelix"],
+                    default=None,
+                    help="instead of the benchmark: Radivik, Gokolix, Larupel, Fubelorn, Zurolorn or Durelix layers of this size ('all': every Radivik "
+                         "size, 'gokolix' / 'larupel' / 'fubelorn' / 'zurolorn' / 'durelix': every size of that design) beside Llama layers of equal size (prefill of --prompt-len tokens, "
                          "decoding at --batch in --context; --layers, default 4, for Radivik)")
-    ap.add_argument("--compare-only", choices=["both", "radivik", "gokolix", "larupel", "fubelorn", "zurolorn", "llama"], default="both")
+    ap.add_argument("--compare-only", choices=["both", "radivik", "gokolix", "larupel", "fubelorn", "zurolorn", "durelix", "llama"], default="both")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")

@@ -550,12 +550,14 @@ def test_linear_swiglu_wide(ops, m, inter):
 
 # -------------------------------------------------------------------- attention
 
-def paged_case(ops, act, hq, hkv, d, lens_new, lens_old, window=None, seed=0, num_blocks=64, poison=1e30, give_back=False):
+def paged_case(ops, act, hq, hkv, d, lens_new, lens_old, window=None, seed=0, num_blocks=64, poison=1e30, give_back=False,
+               sink=None, gated=False, exact_weights=False):
     """Random q/k/v for items with ``old`` cached and ``new`` fresh tokens each, pages from a
     random permutation; returns (kernel output, reference output). Every slot no item writes
     holds ``poison``. ``give_back``: pages wholly in front of the window of an item's first new
     token are not in its table any more (-1, as the cache manager leaves them), and page 0,
-    which stands in for them in the packed table, belongs to nobody and holds ``poison`` too."""
+    which stands in for them in the packed table, belongs to nobody and holds ``poison`` too. ``sink``
+    (float32 [hq]) joins the denominators; ``gated``: outputs times the sigmoid of rows that lie in the middle of wider ones."""
     rng = np.random.default_rng(seed)
     perm = [b for b in rng.permutation(num_blocks).tolist() if not (give_back and b == 0)]
     pk = StepPacker(torch.device(DEV), [GroupMeta(num_blocks, window)], 10, 100000, 8, ops.PREFILL_TILE_Q,
@@ -585,7 +587,9 @@ def paged_case(ops, act, hq, hkv, d, lens_new, lens_old, window=None, seed=0, nu
     qkv = rnd(t, (hq + 2 * hkv) * d, dtype=act, seed=seed + 999)
     out = torch.empty(t, hq * d, dtype=act, device=DEV)
     scale = 1.0 / math.sqrt(d)
-    ops.paged_attention(qkv, out, kv, ctx, 0, hq, hkv, d, scale, window)
+    gate = rnd(t, hq * d + 12, dtype=act, seed=seed + 777) if gated else None
+    ops.paged_attention(qkv, out, kv, ctx, 0, hq, hkv, d, scale, window, exact_weights=exact_weights,
+                        **({} if sink is None else {"sink": sink}), **({"out_gate": (gate, 4)} if gated else {}))
     want = torch.empty(t, hq, d, dtype=torch.float64, device=DEV)
     t0 = 0
     for (k, v), n, old in zip(full, lens_new, lens_old):
@@ -598,8 +602,13 @@ def paged_case(ops, act, hq, hkv, d, lens_new, lens_old, window=None, seed=0, nu
         hide = kpos > qpos
         if window is not None:
             hide = hide | (qpos - kpos >= window)
-        p = torch.softmax(s.masked_fill(hide, float("-inf")), -1)
+        s = s.masked_fill(hide, float("-inf"))
+        if sink is not None:
+            s = torch.cat([s, sink.double()[:, None, None].expand(hq, n, 1)], dim=-1)
+        p = torch.softmax(s, -1)[..., : old + n]
         want[t0:t0 + n] = torch.einsum("hnm,mhd->nhd", p, vv)
+        if gated:
+            want[t0:t0 + n] *= torch.sigmoid(gate[t0:t0 + n, 4: 4 + hq * d].double()).view(n, hq, d)
         t0 += n
     return out.view(t, hq, d), want
 
