@@ -674,6 +674,6 @@ def test_random_configurations_in_both_dtypes(seed, tmp_path):
         rough = plain.PlainDurelix(folder, bf16=True)
         rows = np.concatenate([np.abs(rough.logits(t) - w).max(-1)[:n] / np.abs(w).max(-1)[:n] for t, w, n in zip(reqs, truth, cut)])
         kept = [e for e, (i, p) in zip(errors, (at for exp in expect for at in exp)) if p < cut[i]]
-        assert np.isfinite(errors).all() and len(kept) == len(rows)
-        if len(rows) > 20:
+        assert np.isfinite(errors).all() and len(kept) <= len(rows)
+        if len(kept) > 20:
             check_rows(kept, dtype, (*(float(np.quantile(rows, q)) for q in (0.5, 0.9, 0.99)), 0))
